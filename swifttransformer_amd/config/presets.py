@@ -198,3 +198,34 @@ def pupalix_preset(name: str, **overrides):
                         logit_softcap=30.0, norm_eps=1e-5, max_positions=4096)
     fields.update(overrides)
     return PupalixHyperParam(**fields).validate()
+
+
+# ---- named sizes of the Fiterax family, for runs with random weights: the layer sizes of the OPT model of the same
+# name.  Of every three layers the first is a matrix memory (an eighth of the heads, values of twice the head size), the
+# others grouped attention (a quarter of the heads as key heads, half of each head turned, capped scores); norms in four
+# groups, filters of three taps; every layer has 16 experts of a quarter of the OPT feed-forward's width, 2 a token.
+def fiterax_preset(name: str, **overrides):
+    from .fiterax_param import FiteraxHyperParam
+    key = name.lower().replace("-", "_")
+    size = key.split("_", 1)[1] if "_" in key else ""
+    if "opt_" + size not in _SIZES:
+        raise KeyError(f"invalid model name {name!r}; valid names: " +
+                       " ".join("fiterax_" + k.split("_", 1)[1] for k in _SIZES))
+    n_layers, hidden, heads, ffn = _SIZES["opt_" + size]
+    n_layers = int(overrides.pop("num_layers", n_layers))
+    only = overrides.pop("only", None)            # one mixer type for every layer (measurements)
+    hd = hidden // heads
+    layers = []
+    for i in range(n_layers):
+        kind = only or ("mlstm", "attention", "attention")[i % 3]
+        if kind == "mlstm":
+            mixer = {"heads": max(1, heads // 8), "dim": hd, "vdim": 2 * hd, "gate_cap": 15.0}
+        else:
+            mixer = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": hd, "vdim": hd, "scale": float(hd) ** -0.5,
+                     "softcap": 50.0, "rot": {"dims": hd // 2, "base": 500000.0}}
+        mlp = {"kind": "moe", "router": {"experts": 16, "top": 2, "scale": 2.0}, "expert": {"ff": ffn // 4}}
+        layers.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    fields: Dict = dict(vocab=50272, width=hidden, layers=layers, norm_groups=4, norm_eps=1e-5, taps=3,
+                        embedding_scale=float(hidden) ** 0.5, residual_mult=0.5, max_positions=4096)
+    fields.update(overrides)
+    return FiteraxHyperParam(**fields).validate()

@@ -64,6 +64,16 @@ int st_attn_rows(void* out, float* part_o, float* part_lse, const void* q, int64
                  int num_kv_heads, int head_dim, float scale, int window, float softcap, int num_splits,
                  int num_waves, int dtype, hipStream_t stream);
 
+// The same with a gate: a head's result is multiplied by 1 / (1 + exp(-z)), z the head's logit at head_gate + t *
+// gate_stride for batch row t.  The same for st_attn_prefill_gated.
+int st_attn_rows_gated(void* out, float* part_o, float* part_lse, const void* q, int64_t q_stride,
+                       const void* k_cache, const void* v_cache, int64_t page_stride,
+                       const int* row_ids, const int* token_item, const int* positions,
+                       const int* block_table, const float* head_slopes,
+                       int max_pages, int page_size, int num_tokens, int num_q_heads,
+                       int num_kv_heads, int head_dim, float scale, int window, float softcap, int num_splits,
+                       int num_waves, int dtype, const float* head_gate, int64_t gate_stride, hipStream_t stream);
+
 // No counterpart in the reference.  For callers that cannot allocate (code under HIP graph
 // capture, tight serving loops, harnesses that forbid hipMalloc): st_attn_rows with the key
 // split's partial results kept in a static device array of the library (4 MiB per GPU, held
@@ -88,6 +98,15 @@ int st_attn_prefill(void* out, const void* q, int64_t q_stride,
                     const int* block_table, const float* head_slopes, int max_pages, int page_size,
                     int num_q_heads, int num_kv_heads, int head_dim, float scale, int window, float softcap,
                     int key_split, int tile_rows, int algo, int dtype, hipStream_t stream);
+
+int st_attn_prefill_gated(void* out, const void* q, int64_t q_stride,
+                          const void* k_cache, const void* v_cache, int64_t page_stride,
+                          const int* tile_item, const int* tile_q0, int num_tiles,
+                          const int* item_tok_off, const int* item_start, const int* item_len,
+                          const int* block_table, const float* head_slopes, int max_pages, int page_size,
+                          int num_q_heads, int num_kv_heads, int head_dim, float scale, int window, float softcap,
+                          int key_split, int tile_rows, int algo, int dtype, const float* head_gate, int64_t gate_stride,
+                          hipStream_t stream);
 
 int st_has_attn_prefill();
 int st_attn_prefill_tile_rows(int head_dim, int page_size, int max_pages, int num_q_heads, int num_rows, int dtype);
@@ -212,9 +231,10 @@ int st_latent_write(void* cache, int64_t page_stride, const float* x, int64_t x_
 // the lower index on ties, and their weights: mode 0 the sigmoid of each logit, mode 1 the softmax over
 // the chosen logits alone, mode 2 each chosen expert's share of the softmax over all experts, where only the
 // experts of the `keep` best of `groups` equal groups of neighbours (a group's rank: its largest logit) can be
-// chosen.  Rows whose item is -1 get ids of -1.
-int st_moe_route(int* ids, float* weights, const float* logits, const int* token_item, int num_tokens,
-                 int experts, int top, int mode, int groups, int keep, hipStream_t stream);
+// chosen, mode 3 the sigmoid of each chosen logit over the chosen sigmoids' sum (+ 1e-20), times `scale`, where the
+// choice goes by sigmoid + correction [experts] (else null).  Rows whose item is -1 get ids of -1.
+int st_moe_route(int* ids, float* weights, const float* logits, const int* token_item, const float* correction,
+                 float scale, int num_tokens, int experts, int top, int mode, int groups, int keep, hipStream_t stream);
 // Sorts the num_pairs = tokens * top (token, choice) pairs by expert into tiles of `tile` (16, 64 or 128)
 // places that hold one expert's pairs each: sorted[capacity] (pair index, or -1),
 // place_of_pair[num_pairs] (or -1), tile_expert[capacity / tile] (or -1).
@@ -224,7 +244,8 @@ int st_moe_align(int* sorted, int* place_of_pair, int* tile_expert, const int* i
 // y[place, f] = g * sigmoid(1.702 g) * (u + 1) with g = min(s * (x_t . Wg[e, f]), limit) and
 // u = clamp(s * (x_t . Wu[e, f]), -limit, limit), for the pair (t, j) at `place`, e its expert and s
 // its weight (style 0); style 1: y[place, f] = silu(x_t . Wg[e, f]) * (x_t . Wu[e, f]), no weight and no
-// limit (the weight then multiplies the expert's result, in st_moe_combine).
+// limit (the weight then multiplies the expert's result, in st_moe_combine); style 2: no gate,
+// y[place, f] = gelu(x_t . Wu[e, f]) in its exact form (w_gate is not read).
 // x: [T, width]; w_gate, w_up: [experts, inner, width]; y: [capacity, inner].
 int st_moe_up(void* y, const void* x, const void* w_gate, const void* w_up, const int* sorted,
               const int* tile_expert, const float* weights, int capacity, int tile, int top, int width, int inner,
@@ -283,6 +304,33 @@ int st_qk_norm_write(void* out_q, void* k_cache, void* v_cache, int64_t page_str
                      const float* gain_q, const float* gain_k, const int* token_item, const int* positions,
                      const int* block_table, int max_pages, int page_size, int num_tokens, int heads, int kv_heads,
                      int head_dim, int head_pad, float eps, int write, int dtype, hipStream_t stream);
+
+// ---- root-mean-square norm in groups, alone and with a causal filter over time behind it (csrc/group_norm.hip)
+int st_group_rms(void* out_t, void* out_f32, const float* x, const int* rows, const float* gain, int num_rows, int width,
+                 int groups, float eps, int dtype, hipStream_t stream);
+int st_group_norm_conv(void* out0, const float* gain0, const float* w0, float* state0, int64_t slot_stride0, void* out1,
+                       const float* gain1, const float* w1, float* state1, int64_t slot_stride1, const float* x,
+                       const int* token_item, const int* item_len, const int* item_tok_off, const int* item_slot,
+                       int num_tokens, int num_items, int width, int groups, int taps, float eps, int all_single,
+                       int dtype, hipStream_t stream);
+
+// ---- queries and keys turned and at unit root mean square a head, page write of keys and values (csrc/unit_qk.hip)
+int st_unit_qk_write(void* out_q, void* k_cache, void* v_cache, int64_t page_stride, const float* qkv, int64_t stride,
+                     const float* freq, int half, const float* factor, const int* token_item, const int* positions,
+                     const int* block_table, int max_pages, int page_size, int num_tokens, int heads, int kv_heads,
+                     int key_dim, int value_dim, int pad, float eps, int write, int dtype, hipStream_t stream);
+
+// ---- matrix memory with exponential gates (csrc/matrix_memory.hip)
+int st_memory_step(void* out, const float* proj, int64_t stride, float* state, int64_t slot_stride, const float* bias_i,
+                   const float* bias_f, const float* gain, const int* item_len, const int* item_tok_off,
+                   const int* item_slot, int num_items, int heads, int key_dim, int value_dim, float cap, float q_scale,
+                   float eps, int dtype, hipStream_t stream);
+int st_memory_chunk_rows();
+int st_memory_chunks(void* out, const float* proj, int64_t stride, float* state, int64_t slot_stride, const float* bias_i,
+                     const float* bias_f, const float* gain, const int* item_len, const int* item_tok_off,
+                     const int* item_slot, int num_items, int num_rows, int heads, int key_dim, int value_dim, float cap,
+                     float q_scale, float eps, float* scratch_u, float* scratch_n, double* scratch_s, float* scratch_m,
+                     int64_t scratch_chunks, int dtype, hipStream_t stream);
 
 // Measurement kernels (csrc/probe.hip): a plain streaming read, and a kernel without work.
 int st_probe_read(const void* src, int64_t bytes, void* sink, int workgroups, int pattern, hipStream_t stream);

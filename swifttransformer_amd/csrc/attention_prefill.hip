@@ -59,7 +59,7 @@ __global__ __launch_bounds__(256 * KS, HDP <= 2 ? 4 : 1) void attn_prefill_kerne
     const int* __restrict__ item_tok_off, const int* __restrict__ item_start, const int* __restrict__ item_len,
     const int* __restrict__ block_table, const float* __restrict__ head_slopes, int max_pages, int page_size,
     int page_shift, int num_q_heads, int num_kv_heads, int head_dim, float scale, int window, float softcap,
-    int num_tiles, int deal_period) {
+    int num_tiles, int deal_period, const float* __restrict__ head_gate, int64_t gate_stride) {
     constexpr int KS_STRIDE = 32 * HDP + 8;          // elements between keys of the K block
     extern __shared__ uint4 dyn[];
     constexpr int BUF = PK * KS_STRIDE + (32 * HDP) * VT_STRIDE;   // elements of the block buffer
@@ -409,8 +409,9 @@ __global__ __launch_bounds__(256 * KS, HDP <= 2 ? 4 : 1) void attn_prefill_kerne
     }
     // acc[dt][r] = O[query r16][dim 16dt + 4g + r]
     l = rows4_sum(l);                                // the row's normaliser from its four lanes
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    float inv = l > 0.f ? 1.0f / l : 0.f;
     if (qvalid) {
+        if (head_gate) inv /= 1.f + expf(-head_gate[(int64_t)(row0 + qi) * gate_stride + h]);
         bf16_t* orow = out + ((int64_t)(row0 + qi) * num_q_heads + h) * head_dim;
 #pragma unroll
         for (int dt = 0; dt < 2 * HDP; ++dt) {
@@ -440,7 +441,7 @@ static int launch_prefill(void* out, const void* q, int64_t q_stride, const void
                           const int* item_tok_off, const int* item_start, const int* item_len,
                           const int* block_table, const float* head_slopes, int max_pages, int page_size,
                           int num_q_heads, int num_kv_heads, int head_dim, float scale, int window, float softcap,
-                          hipStream_t stream) {
+                          const float* head_gate, int64_t gate_stride, hipStream_t stream) {
     auto kernel = attn_prefill_kernel<HDP, KS>;
     const size_t lds = prefill_lds(HDP, KS, max_pages);
     if (lds > 48 * 1024) {
@@ -463,7 +464,8 @@ static int launch_prefill(void* out, const void* q, int64_t q_stride, const void
     kernel<<<dim3(num_q_heads, num_tiles), 256 * KS, lds, stream>>>(
         (bf16_t*)out, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, page_stride,
         tile_item, tile_q0, item_tok_off, item_start, item_len, block_table, head_slopes, max_pages, page_size,
-        page_shift, num_q_heads, num_kv_heads, head_dim, scale, window, softcap, num_tiles, deal_period);
+        page_shift, num_q_heads, num_kv_heads, head_dim, scale, window, softcap, num_tiles, deal_period, head_gate,
+        gate_stride);
     ST_LAUNCH_CHECK("attn_prefill");
     return 0;
 }
@@ -487,7 +489,7 @@ int attn_prefill_f32(void* out, const void* q, int64_t q_stride, const void* k_c
                      const int* item_tok_off, const int* item_start, const int* item_len,
                      const int* block_table, const float* head_slopes, int max_pages, int page_size,
                      int num_q_heads, int num_kv_heads, int head_dim, float scale, int window, float softcap,
-                     hipStream_t stream);
+                     const float* head_gate, int64_t gate_stride, hipStream_t stream);
 
 // the direct-load instance (attention_prefill_dma.hip)
 bool attn_prefill_dma_offered(int head_dim, int page_size, int tile_rows, int max_pages);
@@ -512,13 +514,16 @@ using namespace st;
 // tile_rows: 64, or 128 where st_attn_prefill_tile_rows says so (the direct-load kernel only).
 // algo: 0 = chosen here, 1 = the kernel that stages blocks through registers, 2 = the direct-load
 // kernel (an error where it is not offered).
-extern "C" int st_attn_prefill(void* out, const void* q, int64_t q_stride,
+// head_gate (optional): logits of batch row t at head_gate + t * gate_stride, one a head; a head's result is
+// multiplied by their logistic function.
+extern "C" int st_attn_prefill_gated(void* out, const void* q, int64_t q_stride,
                     const void* k_cache, const void* v_cache, int64_t page_stride,
                     const int* tile_item, const int* tile_q0, int num_tiles,
                     const int* item_tok_off, const int* item_start, const int* item_len,
                     const int* block_table, const float* head_slopes, int max_pages, int page_size,
                     int num_q_heads, int num_kv_heads, int head_dim, float scale, int window, float softcap,
-                    int key_split, int tile_rows, int algo, int dtype, hipStream_t stream) {
+                    int key_split, int tile_rows, int algo, int dtype, const float* head_gate, int64_t gate_stride,
+                    hipStream_t stream) {
     ST_CHECK(dtype == kBF16 || dtype == kF32, "attn_prefill: unknown dtype %d", dtype);
     ST_CHECK(num_tiles >= 0 && num_q_heads > 0 && num_kv_heads > 0 && page_size > 0 && max_pages > 0,
              "attn_prefill: bad sizes");
@@ -531,9 +536,9 @@ extern "C" int st_attn_prefill(void* out, const void* q, int64_t q_stride,
     ST_CHECK(scale == scale && scale >= -3.0e38f && scale <= 3.0e38f, "attn_prefill: the score scale must be finite");
     ST_CHECK(tile_rows == 64 || tile_rows == 128, "attn_prefill: tiles of %d rows (64 or 128)", tile_rows);
     ST_CHECK(algo >= 0 && algo <= 2, "attn_prefill: unknown algo %d", algo);
-    // (the direct-load kernel has no score bias, no cap and no chunks: those go through the staging kernel)
+    // (the direct-load kernel has no score bias, no cap, no chunks and no gate: those go through the staging kernel)
     // (and it orders maxima in scaled units, which needs a positive, finite scale)
-    const bool dma_ok = dtype == kBF16 && !head_slopes && softcap == 0.f && window >= 0 && scale > 0.f && scale <= 3.0e38f &&
+    const bool dma_ok = dtype == kBF16 && !head_slopes && !head_gate && softcap == 0.f && window >= 0 && scale > 0.f && scale <= 3.0e38f &&
                         attn_prefill_dma_offered(head_dim, page_size, tile_rows, max_pages);
     ST_CHECK(tile_rows == 64 || (dma_ok && algo != 1),
              "attn_prefill: tiles of 128 rows need the direct-load kernel (bfloat16, head_dim 64 or 128, "
@@ -541,11 +546,12 @@ extern "C" int st_attn_prefill(void* out, const void* q, int64_t q_stride,
              page_size);
     ST_CHECK(algo != 2 || dma_ok, "attn_prefill: the direct-load kernel is not offered for dtype %d head_dim %d "
              "page_size %d%s", dtype, head_dim, page_size, head_slopes ? " with score slopes" : "");
+    ST_CHECK(!head_gate || gate_stride >= num_q_heads, "attn_prefill: a gate has a logit a head");
     if (num_tiles == 0) return 0;
     if (dtype == kF32)
         return attn_prefill_f32(out, q, q_stride, k_cache, v_cache, page_stride, tile_item, tile_q0, num_tiles,
                                 item_tok_off, item_start, item_len, block_table, head_slopes, max_pages, page_size,
-                                num_q_heads, num_kv_heads, head_dim, scale, window, softcap, stream);
+                                num_q_heads, num_kv_heads, head_dim, scale, window, softcap, head_gate, gate_stride, stream);
     ST_CHECK(q_stride % 8 == 0 && ((uintptr_t)q & 15) == 0, "attn_prefill: query rows must be 16-byte aligned");
     const int hdp = (head_dim + 31) / 32;
     // the direct-load kernel wherever it is offered
@@ -560,7 +566,7 @@ extern "C" int st_attn_prefill(void* out, const void* q, int64_t q_stride,
              "attn_prefill: %d wave groups are not offered for head_dim %d", ks, head_dim);
 #define ST_PF(H, S) launch_prefill<H, S>(out, q, q_stride, k_cache, v_cache, page_stride, tile_item, tile_q0, num_tiles, \
         item_tok_off, item_start, item_len, block_table, head_slopes, max_pages, page_size, num_q_heads, num_kv_heads, \
-        head_dim, scale, window, softcap, stream)
+        head_dim, scale, window, softcap, head_gate, gate_stride, stream)
     switch (hdp * 8 + ks) {
         case 1 * 8 + 1: return ST_PF(1, 1);
         case 1 * 8 + 2: return ST_PF(1, 2);
@@ -580,6 +586,19 @@ extern "C" int st_attn_prefill(void* out, const void* q, int64_t q_stride,
         default: return ST_PF(8, 1);
     }
 #undef ST_PF
+}
+
+extern "C" int st_attn_prefill(void* out, const void* q, int64_t q_stride,
+                    const void* k_cache, const void* v_cache, int64_t page_stride,
+                    const int* tile_item, const int* tile_q0, int num_tiles,
+                    const int* item_tok_off, const int* item_start, const int* item_len,
+                    const int* block_table, const float* head_slopes, int max_pages, int page_size,
+                    int num_q_heads, int num_kv_heads, int head_dim, float scale, int window, float softcap,
+                    int key_split, int tile_rows, int algo, int dtype, hipStream_t stream) {
+    return st_attn_prefill_gated(out, q, q_stride, k_cache, v_cache, page_stride, tile_item, tile_q0, num_tiles, item_tok_off,
+                                 item_start, item_len, block_table, head_slopes, max_pages, page_size, num_q_heads,
+                                 num_kv_heads, head_dim, scale, window, softcap, key_split, tile_rows, algo, dtype, nullptr, 0,
+                                 stream);
 }
 
 extern "C" int st_has_attn_prefill() { return 1; }

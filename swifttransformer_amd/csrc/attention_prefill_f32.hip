@@ -36,7 +36,8 @@ __global__ __launch_bounds__(256) void attn_prefill_f32_kernel(
     const int* __restrict__ tile_item, const int* __restrict__ tile_q0,
     const int* __restrict__ item_tok_off, const int* __restrict__ item_start, const int* __restrict__ item_len,
     const int* __restrict__ block_table, const float* __restrict__ head_slopes, int max_pages, int page_size,
-    int num_q_heads, int num_kv_heads, float scale, int window, float softcap, int num_tiles, int deal_period) {
+    int num_q_heads, int num_kv_heads, float scale, int window, float softcap, int num_tiles, int deal_period,
+    const float* __restrict__ head_gate, int64_t gate_stride) {
     constexpr int HD = 16 * DT;
     constexpr int K_STRIDE = HD + 4;                 // floats between keys of the K block
     extern __shared__ uint4 dyn[];
@@ -205,8 +206,9 @@ __global__ __launch_bounds__(256) void attn_prefill_f32_kernel(
     }
     // acc[dt][r] = O[query r16][dim 16dt + 4g + r]
     l = rows4_sum(l);
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    float inv = l > 0.f ? 1.0f / l : 0.f;
     if (qvalid) {
+        if (head_gate) inv /= 1.f + expf(-head_gate[(int64_t)(row0 + qi) * gate_stride + h]);
         float* orow = out + ((int64_t)(row0 + qi) * num_q_heads + h) * HD;
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt)
@@ -221,7 +223,7 @@ int launch(float* out, const float* q, int64_t q_stride, const float* k_cache, c
            int64_t page_stride, const int* tile_item, const int* tile_q0, int num_tiles,
            const int* item_tok_off, const int* item_start, const int* item_len, const int* block_table,
            const float* head_slopes, int max_pages, int page_size, int num_q_heads, int num_kv_heads, float scale,
-           int window, float softcap, hipStream_t stream) {
+           int window, float softcap, const float* head_gate, int64_t gate_stride, hipStream_t stream) {
     constexpr int HD = 16 * DT;
     auto kernel = attn_prefill_f32_kernel<DT>;
     const size_t lds = (size_t)(PK * (HD + 4) + HD * VT_STRIDE) * sizeof(float) + (size_t)max_pages * sizeof(int);
@@ -242,7 +244,7 @@ int launch(float* out, const float* q, int64_t q_stride, const float* k_cache, c
     kernel<<<dim3(num_q_heads, num_tiles), 256, lds, stream>>>(
         out, q, q_stride, k_cache, v_cache, page_stride, tile_item, tile_q0, item_tok_off, item_start, item_len,
         block_table, head_slopes, max_pages, page_size, num_q_heads, num_kv_heads, scale, window, softcap,
-        num_tiles, deal_period);
+        num_tiles, deal_period, head_gate, gate_stride);
     ST_LAUNCH_CHECK("attn_prefill (float)");
     return 0;
 }
@@ -255,11 +257,12 @@ int attn_prefill_f32(void* out, const void* q, int64_t q_stride, const void* k_c
                      const int* item_tok_off, const int* item_start, const int* item_len,
                      const int* block_table, const float* head_slopes, int max_pages, int page_size,
                      int num_q_heads, int num_kv_heads, int head_dim, float scale, int window, float softcap,
-                     hipStream_t stream) {
+                     const float* head_gate, int64_t gate_stride, hipStream_t stream) {
     ST_CHECK(q_stride % 4 == 0 && ((uintptr_t)q & 15) == 0, "attn_prefill: query rows must be 16-byte aligned");
 #define ST_PF(D) case D: return launch<D>((float*)out, (const float*)q, q_stride, (const float*)k_cache,          \
         (const float*)v_cache, page_stride, tile_item, tile_q0, num_tiles, item_tok_off, item_start, item_len,    \
-        block_table, head_slopes, max_pages, page_size, num_q_heads, num_kv_heads, scale, window, softcap, stream)
+        block_table, head_slopes, max_pages, page_size, num_q_heads, num_kv_heads, scale, window, softcap, head_gate, \
+        gate_stride, stream)
     switch (head_dim / 16) {
         ST_PF(1); ST_PF(2); ST_PF(3); ST_PF(4); ST_PF(5); ST_PF(6); ST_PF(7); ST_PF(8);
         ST_PF(9); ST_PF(10); ST_PF(11); ST_PF(12); ST_PF(13); ST_PF(14); ST_PF(15); ST_PF(16);

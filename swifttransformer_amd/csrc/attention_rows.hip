@@ -63,6 +63,9 @@ static int static_scratch(float** ptr) {
 
 typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
 
+// a gate's factor on a head's result, from its logit
+__device__ inline float gate_factor(float z) { return 1.f / (1.f + expf(-z)); }
+
 template <bool ACCURATE>
 __device__ inline float exp_(float x) { return ACCURATE ? expf(x) : __expf(x); }
 
@@ -103,7 +106,8 @@ __global__ __launch_bounds__(512) void attn_rows_kernel(
     const T* __restrict__ k_cache, const T* __restrict__ v_cache, int64_t page_stride,
     const int* __restrict__ row_ids, const int* __restrict__ token_item, const int* __restrict__ positions,
     const int* __restrict__ block_table, const float* __restrict__ head_slopes, int max_pages, int page_size,
-    int num_q_heads, int num_kv_heads, int head_dim, float scale, int window, float softcap, int num_splits) {
+    int num_q_heads, int num_kv_heads, int head_dim, float scale, int window, float softcap, int num_splits,
+    const float* __restrict__ head_gate, int64_t gate_stride) {
     constexpr int VEC = Elem<T>::kVec;
     constexpr int KPW = kWave / LPK;        // keys per wave per step
     const int G = (blockDim.x >> 6) * KPW;  // lane groups in the workgroup (4 or 8 waves)
@@ -279,13 +283,14 @@ __global__ __launch_bounds__(512) void attn_rows_kernel(
     __syncthreads();
     float L = 0.f;
     for (int w = 0; w < nwaves; ++w) L += s_red[8 + w];
+    const float gate = head_gate && num_splits == 1 ? gate_factor(head_gate[(int64_t)t * gate_stride + h]) : 1.f;
     for (int d = threadIdx.x; d < head_dim; d += blockDim.x) {
         float o = 0.f;
 #pragma unroll 4
         for (int i = 0; i < G; ++i) o = fmaf(s_m[i], s_acc[i * head_dim + d], o);
         const float res = L > 0.f ? o / L : 0.f;
         if (num_splits == 1) {
-            Elem<T>::store(out + ((int64_t)t * num_q_heads + h) * head_dim + d, res);
+            Elem<T>::store(out + ((int64_t)t * num_q_heads + h) * head_dim + d, res * gate);
         } else {
             const int64_t pidx = ((int64_t)ri * num_q_heads + h) * num_splits + split;
             part_o[pidx * head_dim + d] = res;
@@ -298,11 +303,13 @@ __global__ __launch_bounds__(512) void attn_rows_kernel(
 template <typename T>
 __global__ __launch_bounds__(64) void attn_merge_kernel(
     T* __restrict__ out, const float* __restrict__ part_o, const float* __restrict__ part_lse,
-    const int* __restrict__ row_ids, int num_q_heads, int head_dim, int num_splits) {
+    const int* __restrict__ row_ids, int num_q_heads, int head_dim, int num_splits, const float* __restrict__ head_gate,
+    int64_t gate_stride) {
     const int64_t row = blockIdx.x;   // ri * num_q_heads + h
     const int64_t ri = row / num_q_heads, h = row - ri * num_q_heads;
     if (row_ids && row_ids[ri] < 0) return;        // padding entry: its partial results were never written
-    const int64_t orow = (int64_t)(row_ids ? row_ids[ri] : ri) * num_q_heads + h;
+    const int64_t t = row_ids ? row_ids[ri] : ri, orow = t * num_q_heads + h;
+    const float gate = head_gate ? gate_factor(head_gate[t * gate_stride + h]) : 1.f;
     const float* lse = part_lse + row * num_splits;
     float M = -INFINITY;
     for (int s = 0; s < num_splits; ++s) M = fmaxf(M, lse[s]);
@@ -318,7 +325,7 @@ __global__ __launch_bounds__(64) void attn_merge_kernel(
                 }
             }
         }
-        Elem<T>::store(out + orow * head_dim + d, W > 0.f ? o / W : 0.f);
+        Elem<T>::store(out + orow * head_dim + d, W > 0.f ? o / W * gate : 0.f);
     }
 }
 
@@ -329,7 +336,7 @@ static int launch_rows(void* out, float* part_o, float* part_lse, const void* q,
                        const int* block_table, const float* head_slopes,
                        int max_pages, int page_size, int num_tokens, int num_q_heads,
                        int num_kv_heads, int head_dim, float scale, int window, float softcap, int num_splits,
-                       int num_waves, hipStream_t stream) {
+                       int num_waves, const float* head_gate, int64_t gate_stride, hipStream_t stream) {
     constexpr int VEC = Elem<T>::kVec;
     const int need = (head_dim + VEC - 1) / VEC;
     int lpk = 1;
@@ -343,7 +350,7 @@ static int launch_rows(void* out, float* part_o, float* part_lse, const void* q,
     attn_rows_kernel<T, L><<<grid, num_waves * 64, lds, stream>>>((T*)out, part_o, part_lse, (const T*)q,  \
         q_stride, (const T*)k_cache, (const T*)v_cache, page_stride, row_ids, token_item, positions, \
         block_table, head_slopes, max_pages, page_size, num_q_heads, num_kv_heads, head_dim, scale, window, \
-        softcap, num_splits)
+        softcap, num_splits, head_gate, gate_stride)
     switch (lpk) {
         case 1: ST_ROWS(1); break;
         case 2: ST_ROWS(2); break;
@@ -358,7 +365,7 @@ static int launch_rows(void* out, float* part_o, float* part_lse, const void* q,
     if (num_splits > 1 && out) {      // without `out` the caller merges the partial results itself
         attn_merge_kernel<T><<<num_tokens * num_q_heads, 64, 0, stream>>>((T*)out, part_o, part_lse,
                                                                           row_ids, num_q_heads, head_dim,
-                                                                          num_splits);
+                                                                          num_splits, head_gate, gate_stride);
         ST_LAUNCH_CHECK("attn_merge");
     }
     return 0;
@@ -377,13 +384,15 @@ using namespace st;
 // part_o [num_tokens*num_q_heads*num_splits*head_dim] and part_lse
 // [num_tokens*num_q_heads*num_splits] floats are needed when num_splits > 1; `out` may then be
 // null: the splits are left unmerged in them (each partial normalised, with its log-sum-exp).
-extern "C" int st_attn_rows(void* out, float* part_o, float* part_lse, const void* q, int64_t q_stride,
+// head_gate (optional): logits of batch row t at head_gate + t * gate_stride, one a head; a head's result is
+// multiplied by their logistic function.
+extern "C" int st_attn_rows_gated(void* out, float* part_o, float* part_lse, const void* q, int64_t q_stride,
                             const void* k_cache, const void* v_cache, int64_t page_stride,
                             const int* row_ids, const int* token_item, const int* positions,
                             const int* block_table, const float* head_slopes,
                             int max_pages, int page_size, int num_tokens, int num_q_heads,
                             int num_kv_heads, int head_dim, float scale, int window, float softcap, int num_splits,
-                            int num_waves, int dtype, hipStream_t stream) {
+                            int num_waves, int dtype, const float* head_gate, int64_t gate_stride, hipStream_t stream) {
     ST_CHECK(num_tokens >= 0 && num_q_heads > 0 && num_kv_heads > 0 && head_dim > 0 && page_size > 0 &&
              max_pages > 0, "attention: bad sizes");
     ST_CHECK(num_q_heads % num_kv_heads == 0, "attention: %d query heads do not divide into %d key heads",
@@ -395,17 +404,30 @@ extern "C" int st_attn_rows(void* out, float* part_o, float* part_lse, const voi
     ST_CHECK(out || num_splits > 1, "attention: no destination");
     ST_CHECK(softcap >= 0.f && softcap <= 3.0e38f, "attention: the cap of the scores must be finite and not negative");
     ST_CHECK(num_waves == 4 || num_waves == 8, "attention: %d waves per workgroup (4 or 8)", num_waves);
+    ST_CHECK(!head_gate || (out && gate_stride >= num_q_heads), "attention: a gate goes with a finished result and a logit a head");
     if (num_tokens == 0) return 0;
     if (dtype == kF32)
         return launch_rows<float>(out, part_o, part_lse, q, q_stride, k_cache, v_cache, page_stride,
                                   row_ids, token_item, positions, block_table, head_slopes, max_pages, page_size, num_tokens,
-                                  num_q_heads, num_kv_heads, head_dim, scale, window, softcap, num_splits, num_waves, stream);
+                                  num_q_heads, num_kv_heads, head_dim, scale, window, softcap, num_splits, num_waves, head_gate, gate_stride, stream);
     if (dtype == kBF16)
         return launch_rows<bf16_t>(out, part_o, part_lse, q, q_stride, k_cache, v_cache, page_stride,
                                    row_ids, token_item, positions, block_table, head_slopes, max_pages, page_size, num_tokens,
-                                   num_q_heads, num_kv_heads, head_dim, scale, window, softcap, num_splits, num_waves, stream);
+                                   num_q_heads, num_kv_heads, head_dim, scale, window, softcap, num_splits, num_waves, head_gate, gate_stride, stream);
     ST_CHECK(false, "attention: unknown dtype %d", dtype);
     return 0;
+}
+
+extern "C" int st_attn_rows(void* out, float* part_o, float* part_lse, const void* q, int64_t q_stride,
+                            const void* k_cache, const void* v_cache, int64_t page_stride,
+                            const int* row_ids, const int* token_item, const int* positions,
+                            const int* block_table, const float* head_slopes,
+                            int max_pages, int page_size, int num_tokens, int num_q_heads,
+                            int num_kv_heads, int head_dim, float scale, int window, float softcap, int num_splits,
+                            int num_waves, int dtype, hipStream_t stream) {
+    return st_attn_rows_gated(out, part_o, part_lse, q, q_stride, k_cache, v_cache, page_stride, row_ids, token_item,
+                              positions, block_table, head_slopes, max_pages, page_size, num_tokens, num_q_heads,
+                              num_kv_heads, head_dim, scale, window, softcap, num_splits, num_waves, dtype, nullptr, 0, stream);
 }
 
 extern "C" int st_attn_rows_static_init() {

@@ -69,9 +69,10 @@ __global__ __launch_bounds__(256) void gemm_tiled_kernel(
             const int n = n0 + tc * 4 + j;
             if (n >= N) continue;
             float v = acc[i][j];
-            if (bias) v += bias[n];
+            if (bias && !ex.bias_unscaled) v += bias[n];
             v = apply_activation(act, v);
             if (ex.out_scale != 0.f) v *= ex.out_scale;
+            if (bias && ex.bias_unscaled) v += bias[n];
             if (residual) v += residual[(int64_t)m * N + n];
             Elem<TO>::store(out + (int64_t)m * N + n, v);
             if (ex.k_cache && n >= ex.q_size) {
@@ -160,6 +161,7 @@ extern "C" int st_gemm(void* out, const void* x, const void* w, const float* bia
     }
     if (ex.out_scale == 1.f) ex.out_scale = 0.f;
     const bool scaled = ex.out_scale != 0.f;
+    ST_CHECK(!ex.bias_unscaled || act == 0, "gemm: a bias behind the factor goes with a product without activation");
     if (M == 0) return 0;
     // the persistent kernel for a few rows and a very wide matrix: float results of a plain product
     const bool wide_can = dtype == kBF16 && out_f32 && !residual && act == 0 && !ex.k_cache && !ex.mg_o && !scaled &&
@@ -193,7 +195,7 @@ extern "C" int st_gemm(void* out, const void* x, const void* w, const float* bia
     // elementwise kernel after the library's product (a product with a residual sum cannot be
     // split like that and stays with the kernels here).
     const bool in_epilogue = activation_in_library(act);
-    const bool library_can = (in_epilogue || !residual) && (!scaled || (act == 0 && !bias));
+    const bool library_can = (in_epilogue || !residual) && (!scaled || (act == 0 && (!bias || ex.bias_unscaled)));
     ST_CHECK(algo != 2 || library_can, "gemm: the library path has no activation %d before a residual sum", act);
     const bool to_library = algo == 2 || (algo == 0 && !ex.ln_x && !ex.mg_o && library_can &&
         (dtype == kF32 || M >= g_library_min_rows ||

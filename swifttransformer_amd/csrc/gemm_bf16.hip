@@ -44,7 +44,7 @@ template <bool OUT_F32>
 __device__ inline void store4(void* out, const float* bias, const float* residual, int act,
                               int m, int n0, int N, floatx4 v, const StGemmExtras& ex) {
     float r[4] = {v[0], v[1], v[2], v[3]};
-    if (bias) {
+    if (bias && !ex.bias_unscaled) {
 #pragma unroll
         for (int i = 0; i < 4; ++i)
             if (n0 + i < N) r[i] += bias[n0 + i];
@@ -53,6 +53,11 @@ __device__ inline void store4(void* out, const float* bias, const float* residua
     if (ex.out_scale != 0.f) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) r[i] *= ex.out_scale;
+    }
+    if (bias && ex.bias_unscaled) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            if (n0 + i < N) r[i] += bias[n0 + i];
     }
     if (residual) {
 #pragma unroll

@@ -58,9 +58,10 @@ extern "C" struct StGemmExtras {
     int* best_idx;
     // scaled result: what the product, bias and activation gave is multiplied by out_scale before
     // the residual is added (0 means 1).  The kernels of gemm.hip and gemm_bf16.hip and the library
-    // (as its alpha, for products without bias and activation) offer it.
+    // (as its alpha, for products without activation, and without bias or with bias_unscaled) offer it.
     float out_scale;
-    int _pad3;
+    // != 0: the bias is added after the factor, out = residual + out_scale * x W^T + bias (no activation)
+    int bias_unscaled;
 };
 
 namespace st {

@@ -2,11 +2,12 @@
 // `experts` small gated feed-forward layers.
 //
 // Everything stays on the device and has a fixed launch shape, so a step can be recorded:
-//   route    per token the `top` largest router logits and the sigmoid of each;
+//   route    per token the `top` best experts and their weights (four rules, see st_moe_route);
 //   align    the (token, choice) pairs sorted by expert into tiles of 16, 64 or 128 places, a tile
 //            holding pairs of one expert only (places left over are marked -1);
 //   up       per tile and 64 inner features: both input products on the matrix cores, rows
-//            gathered through the sorted list, then clamp, gate and product of the two halves;
+//            gathered through the sorted list, then clamp, gate and product of the two halves (experts
+//            without a gate: one product and the exact GELU);
 //   down     per tile and 64 output features: the output product; with one expert a token the
 //            result goes straight into the residual stream, otherwise to a row per pair that
 //   combine  sums in the order of the token's choices.
@@ -15,6 +16,7 @@
 // are bound by the stream of expert weights, which every tile reads once.
 #include "api.h"
 #include "common.h"
+#include "activation.h"
 
 namespace st {
 
@@ -26,8 +28,8 @@ constexpr int kMaxTop = 16;
 
 __global__ __launch_bounds__(256) void moe_route_kernel(
     int* __restrict__ ids, float* __restrict__ weights, const float* __restrict__ logits,
-    const int* __restrict__ token_item, int num_tokens, int experts, int top, int mode, int groups, int keep,
-    int stage) {
+    const int* __restrict__ token_item, const float* __restrict__ correction, float scale, int num_tokens, int experts,
+    int top, int mode, int groups, int keep, int stage) {
     // The rows of the workgroup's tokens go to LDS first, read side by side (a thread that walked its own row in
     // memory would wait for every logit by itself, several times over); rows are experts + 1 floats apart.
     extern __shared__ float s_z[];
@@ -37,7 +39,9 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
         const float* src = logits + (int64_t)t0 * experts;
         for (int i = threadIdx.x; i < n * experts; i += blockDim.x) {
             const int r = i / experts;
-            s_z[r * (experts + 1) + (i - r * experts)] = src[i];
+            // (mode 3 chooses by the sigmoid of a logit plus the expert's correction: formed here, side by side)
+            const float z = src[i];
+            s_z[r * (experts + 1) + (i - r * experts)] = mode == 3 ? 1.f / (1.f + expf(-z)) + correction[i - r * experts] : z;
         }
         __syncthreads();
     }
@@ -74,6 +78,10 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
         for (int e = 0; e < experts; ++e) sum += expf(z[e] - m_all);
         inv_sum = 1.f / sum;
     }
+    // mode 3: what an expert is chosen by, where it was not staged
+    auto choice = [&](int e) {
+        return mode == 3 && !stage ? 1.f / (1.f + expf(-z[e])) + correction[e] : z[e];
+    };
     auto weight_of = [&](float v) { return mode == 0 ? 1.f / (1.f + expf(-v)) : mode == 2 ? expf(v - m_all) * inv_sum : v; };
     if (experts <= 64) {
         // which experts can still be chosen, a bit each: no list of the chosen ones to walk
@@ -88,7 +96,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
             int best = -1;
             float bv = 0.f;
             for (int e = 0; e < experts; ++e) {
-                const float v = z[e];
+                const float v = choice(e);
                 if (((free_ >> e) & 1) && (best < 0 || v > bv)) { best = e; bv = v; }
             }
             free_ &= ~(1ull << best);
@@ -103,7 +111,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
             for (int e = 0; e < experts; ++e) {
                 bool taken = mode == 2 && !((open >> (e / per)) & 1);
                 for (int u = 0; u < j; ++u) taken |= chosen[u] == e;
-                const float v = z[e];
+                const float v = choice(e);
                 if (!taken && (best < 0 || v > bv)) { best = e; bv = v; }
             }
             chosen[j] = best;
@@ -118,6 +126,16 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
         float sum = 0.f;
         for (int j = 0; j < top; ++j) { w[j] = expf(w[j] - m); sum += w[j]; }
         for (int j = 0; j < top; ++j) w[j] /= sum;
+    } else if (mode == 3) {
+        // the chosen experts' sigmoids, without the correction, over their sum
+        float* w = weights + (int64_t)t * top;
+        const float* raw = logits + (int64_t)t * experts;
+        float sum = 0.f;
+        for (int j = 0; j < top; ++j) {
+            w[j] = 1.f / (1.f + expf(-raw[ids[(int64_t)t * top + j]]));
+            sum += w[j];
+        }
+        for (int j = 0; j < top; ++j) w[j] = w[j] / (sum + 1e-20f) * scale;
     }
 }
 
@@ -210,7 +228,8 @@ template <> struct Frag<float> {
 // rows (RT = 1 for few rows an expert, where only the weights' stream counts; RT = 4 or 8 for
 // prompts, where every tile reads its expert's weights again from the L2).
 // Result layout of a block: lane (r16, g) holds rows 4g .. 4g+3 of feature r16.
-template <typename T, int RT>
+// GATED false: one weight matrix (w_up) and the exact GELU of its product (style 2).
+template <typename T, int RT, bool GATED>
 __global__ __launch_bounds__(256) void moe_up_kernel(
     T* __restrict__ y, const T* __restrict__ x, const T* __restrict__ w_gate, const T* __restrict__ w_up,
     const int* __restrict__ sorted, const int* __restrict__ tile_expert, const float* __restrict__ weights,
@@ -230,7 +249,7 @@ __global__ __launch_bounds__(256) void moe_up_kernel(
         p_ok[b] = pair >= 0;
         xr[b] = x + (int64_t)(p_ok[b] ? pair / top : 0) * width;
     }
-    const T* gr = w_gate + ((int64_t)e * inner + (f_ok ? f : 0)) * width;
+    const T* gr = (GATED ? w_gate : w_up) + ((int64_t)e * inner + (f_ok ? f : 0)) * width;
     const T* ur = w_up + ((int64_t)e * inner + (f_ok ? f : 0)) * width;
     floatx4 cg[RT], cu[RT];
 #pragma unroll
@@ -240,13 +259,13 @@ __global__ __launch_bounds__(256) void moe_up_kernel(
     for (int k0 = 0; k0 < width; k0 += D) {
         Frag<T> a[RT], bg, bu;
         const int k = k0 + L * g;
-        bg.load(gr, k, width, f_ok, vec);
+        if (GATED) bg.load(gr, k, width, f_ok, vec);
         bu.load(ur, k, width, f_ok, vec);
 #pragma unroll
         for (int b = 0; b < RT; ++b) a[b].load(xr[b], k, width, p_ok[b], vec);
 #pragma unroll
         for (int b = 0; b < RT; ++b) {
-            cg[b] = Frag<T>::mma(a[b], bg, cg[b]);
+            if (GATED) cg[b] = Frag<T>::mma(a[b], bg, cg[b]);
             cu[b] = Frag<T>::mma(a[b], bu, cu[b]);
         }
     }
@@ -258,7 +277,9 @@ __global__ __launch_bounds__(256) void moe_up_kernel(
             const int place = base + b * kRows + 4 * g + r;
             const int p = sorted[place];
             float out = 0.f;
-            if (p >= 0 && style == 1) {
+            if (p >= 0 && !GATED) {
+                out = apply_activation(kActGeluErf, cu[b][r]);
+            } else if (p >= 0 && style == 1) {
                 const float gv = cg[b][r];
                 out = gv / (1.f + expf(-gv)) * cu[b][r];
             } else if (p >= 0) {
@@ -330,12 +351,15 @@ __global__ __launch_bounds__(256) void moe_down_kernel(
 typedef float floatx16 __attribute__((ext_vector_type(16)));
 __device__ inline int rot(int row, int chunk) { return row * 8 + (chunk ^ ((row >> 1) & 7)); }
 
-template <bool UP>
+// GELU: as UP, but the 128 weight rows are 128 inner features of the one input matrix of experts without a gate.
+enum TiledKind : int { kTiledDown = 0, kTiledUp = 1, kTiledGelu = 2 };
+template <int KIND>
 __global__ __launch_bounds__(256) void moe_tiled_kernel(
     bf16_t* __restrict__ y_out, float* __restrict__ out, const float* __restrict__ residual,
     float* __restrict__ pair_out, const bf16_t* __restrict__ a_rows, const bf16_t* __restrict__ w0,
     const bf16_t* __restrict__ w1, const int* __restrict__ sorted, const int* __restrict__ tile_expert,
     const float* __restrict__ weights, int top, int N, int K, float limit, float out_scale, int style) {
+    constexpr bool UP = KIND == kTiledUp, GATHER = KIND != kTiledDown;
     __shared__ uint4 sw[128 * 8];      // weight rows: [row][chunk of 8 in depth]
     __shared__ uint4 sx[128 * 8];      // places
     const int tile = blockIdx.x;
@@ -357,7 +381,7 @@ __global__ __launch_bounds__(256) void moe_tiled_kernel(
         else { n = n0 + row; m = w0; }
         wrow[i] = n < N ? m + ((int64_t)e * N + n) * K : nullptr;
         const int p = sorted[base + row];
-        xrow[i] = UP ? (p >= 0 ? a_rows + (int64_t)(p / top) * K : nullptr) : a_rows + (int64_t)(base + row) * K;
+        xrow[i] = GATHER ? (p >= 0 ? a_rows + (int64_t)(p / top) * K : nullptr) : a_rows + (int64_t)(base + row) * K;
     }
     floatx16 acc[2][2];
 #pragma unroll
@@ -435,6 +459,21 @@ __global__ __launch_bounds__(256) void moe_tiled_kernel(
                 else
                     for (int u = 0; u < 4 && f + u < N; ++u) Elem<bf16_t>::store(dst + u, r[u]);
             }
+        } else if (KIND == kTiledGelu) {
+#pragma unroll
+            for (int i = 0; i < 2; ++i)
+#pragma unroll
+                for (int q4 = 0; q4 < 4; ++q4) {
+                    const int f = n0 + wn * 64 + i * 32 + 8 * q4 + 4 * lh;
+                    if (f >= N) continue;
+                    float r[4];
+#pragma unroll
+                    for (int u = 0; u < 4; ++u) r[u] = p >= 0 ? apply_activation(kActGeluErf, acc[i][j][4 * q4 + u]) : 0.f;
+                    bf16_t* dst = y_out + (int64_t)place * N + f;
+                    if (f + 3 < N && (N & 3) == 0) Elem<bf16_t>::store4(dst, r);
+                    else
+                        for (int u = 0; u < 4 && f + u < N; ++u) Elem<bf16_t>::store(dst + u, r[u]);
+                }
         } else {
             if (p < 0) continue;
 #pragma unroll
@@ -483,10 +522,12 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(
 
 using namespace st;
 
-extern "C" int st_moe_route(int* ids, float* weights, const float* logits, const int* token_item, int num_tokens,
-                            int experts, int top, int mode, int groups, int keep, hipStream_t stream) {
-    ST_CHECK(mode >= 0 && mode <= 2, "moe_route: mode 0 (sigmoid of each), 1 (softmax over the chosen) or 2 (softmax "
-             "over all, the choice within the best groups)");
+extern "C" int st_moe_route(int* ids, float* weights, const float* logits, const int* token_item, const float* correction,
+                            float scale, int num_tokens, int experts, int top, int mode, int groups, int keep,
+                            hipStream_t stream) {
+    ST_CHECK(mode >= 0 && mode <= 3, "moe_route: mode 0 (sigmoid of each), 1 (softmax over the chosen), 2 (softmax "
+             "over all, the choice within the best groups) or 3 (sigmoids over their sum, a corrected choice)");
+    ST_CHECK(mode != 3 || correction, "moe_route: mode 3 chooses by corrected scores");
     if (mode != 2) groups = keep = 1;
     ST_CHECK(groups >= 1 && groups <= 64 && experts % groups == 0 && keep >= 1 && keep <= groups,
              "moe_route: %d experts in %d groups of which %d are kept (up to 64 equal groups)", experts, groups, keep);
@@ -502,7 +543,7 @@ extern "C" int st_moe_route(int* ids, float* weights, const float* logits, const
     const int threads = 256 * row <= 48 * 1024 ? 256 : 64;
     const int stage = threads * row <= 48 * 1024;
     moe_route_kernel<<<(num_tokens + threads - 1) / threads, threads, stage ? threads * row : 0, stream>>>(
-        ids, weights, logits, token_item, num_tokens, experts, top, mode, groups, keep, stage);
+        ids, weights, logits, token_item, correction, scale, num_tokens, experts, top, mode, groups, keep, stage);
     ST_LAUNCH_CHECK("moe_route");
     return 0;
 }
@@ -531,7 +572,8 @@ extern "C" int st_moe_up(void* y, const void* x, const void* w_gate, const void*
                          const int* tile_expert, const float* weights, int capacity, int tile, int top, int width,
                          int inner, float limit, int style, int dtype, hipStream_t stream) {
     const int kTile = tile;
-    ST_CHECK(style == 0 || style == 1, "moe_up: style 0 (weighted, clamped inputs) or 1 (plain gated unit)");
+    ST_CHECK(style >= 0 && style <= 2, "moe_up: style 0 (weighted, clamped inputs), 1 (plain gated unit) or 2 (no gate, GELU)");
+    if (style == 2) w_gate = w_up;
     ST_CHECK(tile == 16 || tile == 64 || tile == 128, "moe_up: tiles of 16, 64 or 128 places, not %d", tile);
     ST_CHECK(capacity > 0 && capacity % kTile == 0 && top >= 1 && width > 0 && inner > 0, "moe_up: bad sizes");
     ST_CHECK(y && x && w_gate && w_up && sorted && tile_expert && weights, "moe_up: null operand");
@@ -539,19 +581,27 @@ extern "C" int st_moe_up(void* y, const void* x, const void* w_gate, const void*
     ST_CHECK(grid.y <= 65535, "moe_up: too many inner features");
     const int vec = rows_vectorised(x, w_gate, w_up, width, dtype);
     if (dtype == kBF16 && tile == 128 && vec) {
+        if (style == 2) {
+            moe_tiled_kernel<kTiledGelu><<<dim3(capacity / 128, (inner + 127) / 128), 256, 0, stream>>>((bf16_t*)y, nullptr, nullptr,
+                nullptr, (const bf16_t*)x, (const bf16_t*)w_up, nullptr, sorted, tile_expert, weights, top, inner, width, limit, 1.f, style);
+            ST_LAUNCH_CHECK("moe_up (tiled, no gate)");
+            return 0;
+        }
         const dim3 g2(capacity / 128, (inner + 63) / 64);
-        moe_tiled_kernel<true><<<g2, 256, 0, stream>>>((bf16_t*)y, nullptr, nullptr, nullptr, (const bf16_t*)x,
+        moe_tiled_kernel<kTiledUp><<<g2, 256, 0, stream>>>((bf16_t*)y, nullptr, nullptr, nullptr, (const bf16_t*)x,
             (const bf16_t*)w_gate, (const bf16_t*)w_up, sorted, tile_expert, weights, top, inner, width, limit, 1.f, style);
         ST_LAUNCH_CHECK("moe_up (tiled)");
         return 0;
     }
-#define ST_UP(T, RT)                                                                                         \
-    moe_up_kernel<T, RT><<<grid, 256, 0, stream>>>((T*)y, (const T*)x, (const T*)w_gate, (const T*)w_up, sorted, \
-                                                   tile_expert, weights, top, width, inner, limit, style, vec)
+#define ST_UP_G(T, RT, G)                                                                                    \
+    moe_up_kernel<T, RT, G><<<grid, 256, 0, stream>>>((T*)y, (const T*)x, (const T*)w_gate, (const T*)w_up, sorted, \
+                                                      tile_expert, weights, top, width, inner, limit, style, vec)
+#define ST_UP(T, RT) do { if (style == 2) ST_UP_G(T, RT, false); else ST_UP_G(T, RT, true); } while (0)
     if (dtype == kF32) { if (tile == 16) ST_UP(float, 1); else if (tile == 64) ST_UP(float, 4); else ST_UP(float, 8); }
     else if (dtype == kBF16) { if (tile == 16) ST_UP(bf16_t, 1); else if (tile == 64) ST_UP(bf16_t, 4); else ST_UP(bf16_t, 8); }
     else ST_CHECK(false, "moe_up: unknown dtype %d", dtype);
 #undef ST_UP
+#undef ST_UP_G
     ST_LAUNCH_CHECK("moe_up");
     return 0;
 }
@@ -570,7 +620,7 @@ extern "C" int st_moe_down(float* out, const float* residual, float* pair_out, c
     const int vec = rows_vectorised(y, w_down, w_down, inner, dtype);
     if (dtype == kBF16 && tile == 128 && vec) {
         const dim3 g2(capacity / 128, (width + 127) / 128);
-        moe_tiled_kernel<false><<<g2, 256, 0, stream>>>(nullptr, out, residual, pair_out, (const bf16_t*)y,
+        moe_tiled_kernel<kTiledDown><<<g2, 256, 0, stream>>>(nullptr, out, residual, pair_out, (const bf16_t*)y,
             (const bf16_t*)w_down, nullptr, sorted, tile_expert, nullptr, top, width, inner, 0.f, out_scale, 0);
         ST_LAUNCH_CHECK("moe_down (tiled)");
         return 0;

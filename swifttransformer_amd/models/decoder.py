@@ -30,10 +30,11 @@ class Layer:
     mixer_out_norm: object = None
     ffn_out_norm: object = None
     side_input: object = None
+    ffn_conv: object = None
 
     def parts(self):
         return tuple(p for p in (self.arrangement, self.mixer_norm, self.mixer_conv, self.mixer, self.mixer_out_norm, self.ffn_norm,
-                                 self.feed_forward, self.ffn_out_norm, self.side_input) if p is not None)
+                                 self.ffn_conv, self.feed_forward, self.ffn_out_norm, self.side_input) if p is not None)
 
 
 EMBEDDING_CACHE = ("embedding",)     # the cache id of what an embedding part keeps a request (its last token)
@@ -43,6 +44,11 @@ def conv_cache_id(run: int):
     """The cache id of the state that the ``mixer_conv`` part of the schedule's ``run``-th entry
     keeps: one per run of a layer, also where the run's mixer reads another run's cache."""
     return (run, "mixer_conv")
+
+
+def ffn_conv_cache_id(run: int):
+    """The same for the ``ffn_conv`` part."""
+    return (run, "ffn_conv")
 
 
 class DecoderModel:
@@ -69,7 +75,8 @@ class DecoderModel:
                 mixer_conv=opt("token_conv", getattr(ls, "mixer_conv", None)),
                 mixer_out_norm=opt("norm", getattr(ls, "mixer_out_norm", None)),
                 ffn_out_norm=opt("norm", getattr(ls, "ffn_out_norm", None)),
-                side_input=opt("side_input", getattr(ls, "side_input", None)))
+                side_input=opt("side_input", getattr(ls, "side_input", None)),
+                ffn_conv=opt("token_conv", getattr(ls, "ffn_conv", None)))
             needs = getattr(layer.arrangement, "needs", ())
             missing = [n for n in needs if getattr(layer, n) is None]
             if missing:
@@ -118,7 +125,8 @@ class DecoderModel:
     # -------------------------------------------------------------------- cache
     def cache_needs(self) -> Dict[int, CacheNeed]:
         """cache id -> need, for every cache the schedule writes: the mixers' under the schedule's
-        own ids (integers), the state of a run's ``mixer_conv`` part under ``conv_cache_id(run)``."""
+        own ids (integers), the states of a run's ``mixer_conv`` and ``ffn_conv`` parts under
+        ``conv_cache_id(run)`` and ``ffn_conv_cache_id(run)``."""
         needs: Dict[object, CacheNeed] = {}
         if hasattr(self.embedding, "cache_need") and self.embedding.cache_need() is not None:
             needs[EMBEDDING_CACHE] = self.embedding.cache_need()
@@ -126,6 +134,8 @@ class DecoderModel:
             layer = self.layers[e.layer]
             if layer.mixer_conv is not None:
                 needs[conv_cache_id(run)] = layer.mixer_conv.cache_need()
+            if layer.ffn_conv is not None:
+                needs[ffn_conv_cache_id(run)] = layer.ffn_conv.cache_need()
             if hasattr(layer.mixer, "cache_parts"):
                 # a mixer of several caches: each under (the run's cache id, the mixer's name for it)
                 if not e.write:
@@ -190,7 +200,10 @@ class DecoderModel:
                 cache = {name: caches.get((e.cache, name)) for name in layer.mixer.cache_parts()}
             else:
                 cache = caches.get(e.cache)
-            if layer.mixer_conv is not None:
+            if layer.ffn_conv is not None:
+                x32 = layer.arrangement.forward(x32, layer, ctx, cache, e.write, conv_cache=caches.get(conv_cache_id(run)),
+                                                ffn_conv_cache=caches.get(ffn_conv_cache_id(run)))
+            elif layer.mixer_conv is not None:
                 x32 = layer.arrangement.forward(x32, layer, ctx, cache, e.write,
                                                 conv_cache=caches.get(conv_cache_id(run)))
             elif getattr(layer.arrangement, "reads_ahead", False):

@@ -53,12 +53,12 @@ def _lib():
         lib.st_gemm_wide_offered.argtypes = [_c_int, _c_int, _c_int, _c_int]
         lib.st_gemm_can_fuse_merge.argtypes = [_c_int] * 7
         lib.st_gemm_library_tuning.argtypes = [_c_int]
-        lib.st_attn_rows.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_i64, _c_p, _c_p, _c_i64, _c_p, _c_p, _c_p,
-                                     _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f, _c_int, _c_f, _c_int,
-                                     _c_int, _c_int, _c_p]
-        lib.st_attn_prefill.argtypes = [_c_p, _c_p, _c_i64, _c_p, _c_p, _c_i64, _c_p, _c_p, _c_int,
-                                        _c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_int,
-                                        _c_f, _c_int, _c_f, _c_int, _c_int, _c_int, _c_int, _c_p]
+        lib.st_attn_rows_gated.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_i64, _c_p, _c_p, _c_i64, _c_p, _c_p, _c_p,
+                                           _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f, _c_int, _c_f,
+                                           _c_int, _c_int, _c_int, _c_p, _c_i64, _c_p]
+        lib.st_attn_prefill_gated.argtypes = [_c_p, _c_p, _c_i64, _c_p, _c_p, _c_i64, _c_p, _c_p, _c_int,
+                                              _c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_int,
+                                              _c_f, _c_int, _c_f, _c_int, _c_int, _c_int, _c_int, _c_p, _c_i64, _c_p]
         lib.st_attn_prefill_tile_rows.argtypes = [_c_int] * 6
         lib.st_probe_read.argtypes = [_c_p, _c_i64, _c_p, _c_int, _c_int, _c_p]
         lib.st_probe_empty.argtypes = [_c_p, _c_p]
@@ -92,7 +92,7 @@ def _lib():
                                            _c_f, _c_int, _c_p]
         lib.st_latent_write.argtypes = [_c_p, _c_i64, _c_p, _c_i64, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int,
                                         _c_int, _c_int, _c_f, _c_int, _c_p, _c_f, _c_int, _c_p]
-        lib.st_moe_route.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_p]
+        lib.st_moe_route.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_p, _c_f, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_p]
         lib.st_moe_align.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_p]
         lib.st_moe_up.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_int,
                                   _c_f, _c_int, _c_int, _c_p]
@@ -118,6 +118,16 @@ def _lib():
                                         _c_int, _c_i64, _c_i64, _c_f, _c_int, _c_int, _c_p]
         lib.st_qk_norm_write.argtypes = [_c_p, _c_p, _c_p, _c_i64, _c_p, _c_i64, _c_p, _c_p, _c_p, _c_p, _c_p, _c_int,
                                          _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f, _c_int, _c_int, _c_p]
+        lib.st_group_rms.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_f, _c_int, _c_p]
+        lib.st_group_norm_conv.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_i64, _c_p, _c_p, _c_p, _c_p, _c_i64, _c_p, _c_p, _c_p,
+                                           _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f, _c_int, _c_int, _c_p]
+        lib.st_unit_qk_write.argtypes = [_c_p, _c_p, _c_p, _c_i64, _c_p, _c_i64, _c_p, _c_int, _c_p, _c_p, _c_p, _c_p, _c_int,
+                                         _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f, _c_int, _c_int, _c_p]
+        lib.st_memory_step.argtypes = [_c_p, _c_p, _c_i64, _c_p, _c_i64, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int,
+                                       _c_int, _c_int, _c_f, _c_f, _c_f, _c_int, _c_p]
+        lib.st_memory_chunks.argtypes = [_c_p, _c_p, _c_i64, _c_p, _c_i64, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int,
+                                         _c_int, _c_int, _c_int, _c_f, _c_f, _c_f, _c_p, _c_p, _c_p, _c_p, _c_i64, _c_int,
+                                         _c_p]
         if torch.cuda.is_available():
             lib.st_gemm_library_init()  # handle and workspace exist before any stream capture
         _configured = True
@@ -279,7 +289,7 @@ class _GemmExtras(ctypes.Structure):
                 ("mg_o", _c_p), ("mg_lse", _c_p), ("mg_splits", _c_int), ("mg_heads", _c_int),
                 ("mg_head_dim", _c_int), ("_pad2", _c_int),
                 ("ln_rows", _c_p), ("best_ids", _c_p), ("best_val", _c_p), ("best_idx", _c_p),
-                ("out_scale", _c_f), ("_pad3", _c_int)]
+                ("out_scale", _c_f), ("bias_unscaled", _c_int)]
 
 
 class KvScatter:
@@ -382,7 +392,7 @@ ACTIVATIONS = {"none": 0, "relu": 1, "silu": 2, "gelu_tanh": 3, "gelu_new": 3, "
 
 
 def _d_gemm(x, w, *, bias=None, residual=None, activation="none", out=None, out_f32=False, algo=0,
-            kv_scatter=None, best=None, out_scale=1.0):
+            kv_scatter=None, best=None, out_scale=1.0, bias_unscaled=False):
     N, K = w.shape
     fused = []
     if isinstance(x, NormInput):
@@ -413,9 +423,10 @@ def gemm(x, w: torch.Tensor, *, bias: Optional[torch.Tensor] = None,
          residual: Optional[torch.Tensor] = None, activation: str = "none",
          out: Optional[torch.Tensor] = None, out_f32: bool = False, algo: int = 0,
          kv_scatter: Optional[KvScatter] = None, best: Optional[torch.Tensor] = None,
-         out_scale: float = 1.0) -> torch.Tensor:
+         out_scale: float = 1.0, bias_unscaled: bool = False) -> torch.Tensor:
     """out[M,N] = out_scale * act(x[M,K] @ w[N,K]^T (+bias)) (+residual); float accumulation.
-    ``activation`` is one of ``ACTIVATIONS``.
+    ``activation`` is one of ``ACTIVATIONS``.  ``bias_unscaled`` (no activation): the bias is added behind the factor,
+    which is the order the vendor library knows (a caller multiplies the bias itself).
 
     ``x`` is a tensor of w's dtype, a ``NormInput`` (where ``can_fuse_norm``) or a
     ``SplitAttention`` (where ``can_fuse_merge``).  With
@@ -490,6 +501,7 @@ def gemm(x, w: torch.Tensor, *, bias: Optional[torch.Tensor] = None,
         if ex is None:
             ex = _GemmExtras()
         ex.out_scale = float(out_scale)
+        ex.bias_unscaled = int(bool(bias_unscaled))
     _check(_lib().st_gemm(_ptr(out), x_ptr, _ptr(w), _ptr(bias), _ptr(residual), M, N, K, ACTIVATIONS[activation],
                           code, int(odt == torch.float32), int(algo),
                           ctypes.byref(ex) if ex is not None else None, _stream()))
@@ -563,13 +575,24 @@ def _d_attention_prefill(q, k_cache, v_cache, tile_item, *a, **kw):
     return info
 
 
+def _gate_rows(head_gate: Optional[torch.Tensor], rows: int, heads: int) -> int:
+    """The row stride of a gate's logits (0: no gate)."""
+    if head_gate is None:
+        return 0
+    _need(head_gate, "head_gate", torch.float32, (rows, heads), contiguous=False)
+    if head_gate.stride(1) != 1 and heads > 1:
+        raise KernelError("head_gate: rows must be dense")
+    return max(head_gate.stride(0), heads)
+
+
 @_timed("attention_rows", _d_attention_rows)
 def attention_rows(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                    token_item: torch.Tensor, positions: torch.Tensor, block_table: torch.Tensor,
                    num_q_heads: int, scale: float, *, window: int = 0, num_splits: int = 1,
                    num_waves: int = 4, row_ids: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None,
                    workspace: Optional[torch.Tensor] = None, merge: bool = True,
-                   head_slopes: Optional[torch.Tensor] = None, softcap: float = 0.0):
+                   head_slopes: Optional[torch.Tensor] = None, softcap: float = 0.0,
+                   head_gate: Optional[torch.Tensor] = None):
     """Each query row attends over its request's cached keys [lo, position].
 
     q: [T, num_q_heads*head_dim] view (row stride free).  Returns [T, num_q_heads*head_dim];
@@ -578,7 +601,9 @@ def attention_rows(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
     ``SplitAttention`` for a product to merge.  ``head_slopes`` (float32 [num_q_heads]): a head's
     scaled scores get slope * (key position - query position) added.  ``window`` > 0: a row reads the last
     ``window`` positions; < 0: the positions of its own chunk of ``-window`` positions, chunks counted from
-    the sequence's start.  ``softcap`` > 0: scaled scores pass through softcap * tanh(score / softcap)."""
+    the sequence's start.  ``softcap`` > 0: scaled scores pass through softcap * tanh(score / softcap).
+    ``head_gate`` (float [T, num_q_heads], dense rows of any stride): a head's result is multiplied by
+    sigmoid(head_gate[t, head])."""
     num_pages, nkv, ps, hd = _check_cache(k_cache, v_cache, q)
     T = q.shape[0]
     if head_slopes is not None:
@@ -595,6 +620,9 @@ def attention_rows(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
         if out is None:
             out = empty((T, num_q_heads * hd), q.dtype, q.device)
         _need(out, "out", q.dtype, (T, num_q_heads * hd))
+    if head_gate is not None and not merge:
+        raise KernelError("a gate goes with a merged result")
+    gate_stride = _gate_rows(head_gate, T, num_q_heads)
     n_rows = T
     if row_ids is not None:
         n_rows = row_ids.shape[0]
@@ -619,12 +647,13 @@ def attention_rows(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
             o_ptr, q_ptr = (out[r0:r1].data_ptr() if merge else None), q[r0:r1].data_ptr()
             ti_ptr, po_ptr = token_item[r0:r1].data_ptr(), positions[r0:r1].data_ptr()
             rid_ptr = None
-        _check(_lib().st_attn_rows(
+        g_ptr = None if head_gate is None else (head_gate if row_ids is not None else head_gate[r0:r1]).data_ptr()
+        _check(_lib().st_attn_rows_gated(
             o_ptr, _ptr(part_o), _ptr(part_lse), q_ptr, q.stride(0),
             _ptr(k_cache), _ptr(v_cache), k_cache.stride(0), rid_ptr, ti_ptr, po_ptr,
             _ptr(block_table), _ptr(head_slopes), block_table.shape[1], ps, r1 - r0,
             num_q_heads, nkv, hd, float(scale), int(window), float(softcap), int(num_splits), int(num_waves),
-            dtype_code(q.dtype), _stream()))
+            dtype_code(q.dtype), g_ptr, gate_stride, _stream()))
     if not merge:
         return SplitAttention(part_o.view(T, num_q_heads, num_splits, hd), part_lse.view(T, num_q_heads, num_splits))
     return out
@@ -637,7 +666,8 @@ def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
                       block_table: torch.Tensor, num_q_heads: int, scale: float, *,
                       window: int = 0, out: Optional[torch.Tensor] = None, key_split: int = 0,
                       tile_rows: int = 64, algo: int = 0,
-                      head_slopes: Optional[torch.Tensor] = None, softcap: float = 0.0) -> torch.Tensor:
+                      head_slopes: Optional[torch.Tensor] = None, softcap: float = 0.0,
+                      head_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Tiles of consecutive query rows of prompt portions attend over the cache.
 
     Tile i covers rows [tile_q0[i], tile_q0[i]+tile_rows) of item tile_item[i]; row r of an
@@ -645,8 +675,8 @@ def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
     ``key_split``: groups of waves that share a tile's key blocks (1, 2 or 4; 0: chosen from
     the number of tiles).  ``tile_rows``: 64, or 128 where ``prefill_tile_rows`` says so.
     ``algo``: 0 chosen by the library, 1 the kernel that stages key blocks through registers,
-    2 the kernel that loads them straight into LDS (it takes no ``head_slopes``, no ``softcap`` and no
-    negative ``window``, which are as in ``attention_rows``)."""
+    2 the kernel that loads them straight into LDS (it takes no ``head_slopes``, no ``softcap``, no ``head_gate``
+    and no negative ``window``, which are as in ``attention_rows``)."""
     num_pages, nkv, ps, hd = _check_cache(k_cache, v_cache, q)
     T = q.shape[0]
     _need(q, "q", None, (T, num_q_heads * hd), contiguous=False)
@@ -663,11 +693,13 @@ def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
     _need(out, "out", q.dtype, (T, num_q_heads * hd))
     if head_slopes is not None:
         _need(head_slopes, "head_slopes", torch.float32, (num_q_heads,))
-    _check(_lib().st_attn_prefill(
+    gate_stride = _gate_rows(head_gate, T, num_q_heads)
+    _check(_lib().st_attn_prefill_gated(
         _ptr(out), _ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache), k_cache.stride(0),
         _ptr(tile_item), _ptr(tile_q0), nt, _ptr(item_tok_off), _ptr(item_start), _ptr(item_len),
         _ptr(block_table), _ptr(head_slopes), block_table.shape[1], ps, num_q_heads, nkv, hd, float(scale), int(window),
-        float(softcap), int(key_split), int(tile_rows), int(algo), dtype_code(q.dtype), _stream()))
+        float(softcap), int(key_split), int(tile_rows), int(algo), dtype_code(q.dtype), _ptr(head_gate), gate_stride,
+        _stream()))
     return out
 
 
@@ -1236,17 +1268,19 @@ def moe_capacity(num_tokens: int, top: int, experts: int, tile: int) -> int:
 
 def _d_moe(x, logits, w_gate, w_up, w_down, residual, *, top, limit=0.0, out_scale=1.0, token_item=None, **kw):
     T, W = x.shape
-    E, F, _ = w_gate.shape
+    E, F, _ = w_up.shape
     used = min(E, T * top)
-    return {"rows": T, "width": W, "inner": F, "experts": E, "top": top,
-            "flops": 6 * T * top * W * F, "bytes": used * 3 * F * W * x.element_size() + T * W * (x.element_size() + 8)}
+    mats = 3 if w_gate is not None else 2
+    return {"rows": T, "width": W, "inner": F, "experts": E, "top": top, "flops": 2 * mats * T * top * W * F,
+            "bytes": used * mats * F * W * x.element_size() + T * W * (x.element_size() + 8)}
 
 
 @_timed("routed_experts", _d_moe)
-def routed_experts(x: torch.Tensor, logits: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor,
+def routed_experts(x: torch.Tensor, logits: torch.Tensor, w_gate: Optional[torch.Tensor], w_up: torch.Tensor,
                    w_down: torch.Tensor, residual: Optional[torch.Tensor], *, top: int, limit: float = 0.0,
                    out_scale: float = 1.0, token_item: Optional[torch.Tensor] = None,
-                   style: str = "scaled_input", groups: int = 1, keep: int = 1) -> torch.Tensor:
+                   style: str = "scaled_input", groups: int = 1, keep: int = 1,
+                   correction: Optional[torch.Tensor] = None, scale: float = 1.0) -> torch.Tensor:
     """residual <- residual + out_scale * sum over a row's ``top`` best experts e (by ``logits``) of
     Wd[e] y with y = g * sigmoid(1.702 g) * (u + 1), g = min(s * Wg[e] x, limit),
     u = clamp(s * Wu[e] x, -limit, limit), s = sigmoid(logit of e).  In place on ``residual``
@@ -1258,20 +1292,29 @@ def routed_experts(x: torch.Tensor, logits: torch.Tensor, w_gate: torch.Tensor, 
     ``style`` "softmax_all": the same experts, weighted by their shares of the softmax over all experts' logits
     (not renormalised); only experts of the ``keep`` best of ``groups`` equal groups of neighbours can be chosen,
     a group ranking by its largest logit.
+    ``style`` "sigmoid_output": a row's experts are those with the largest sigmoid(logit) + ``correction`` (float
+    [experts]), weighted by scale * sigmoid(logit) / (the chosen sigmoids' sum + 1e-20).
+
+    ``w_gate`` None (not in the first style): experts without a gate, Wd[e] gelu(Wu[e] x), the exact GELU.
 
     x: [T, width]; logits: float [T, experts]; w_gate, w_up: [experts, inner, width]; w_down:
     [experts, width, inner].  Rows whose ``token_item`` is negative are left as they are."""
     T, W = x.shape
-    E, F, _ = w_gate.shape
-    _need(x, "x", w_gate.dtype, (T, W))
+    E, F, _ = w_up.shape
+    _need(x, "x", w_up.dtype, (T, W))
     _need(logits, "logits", torch.float32, (T, E))
-    _need(w_gate, "w_gate", None, (E, F, W))
-    _need(w_up, "w_up", w_gate.dtype, (E, F, W))
-    _need(w_down, "w_down", w_gate.dtype, (E, W, F))
-    if style not in ("scaled_input", "softmax_output", "softmax_all"):
+    if w_gate is not None:
+        _need(w_gate, "w_gate", w_up.dtype, (E, F, W))
+    _need(w_up, "w_up", None, (E, F, W))
+    _need(w_down, "w_down", w_up.dtype, (E, W, F))
+    if style not in ("scaled_input", "softmax_output", "softmax_all", "sigmoid_output"):
         raise KernelError(f"routed_experts: unknown style {style!r}")
     on_output = style != "scaled_input"
-    mode = {"scaled_input": 0, "softmax_output": 1, "softmax_all": 2}[style]
+    mode = {"scaled_input": 0, "softmax_output": 1, "softmax_all": 2, "sigmoid_output": 3}[style]
+    if w_gate is None and not on_output:
+        raise KernelError("routed_experts: this style has gated experts")
+    if mode == 3:
+        _need(correction, "correction", torch.float32, (E,))
     if mode == 2 and (groups < 1 or E % groups or not 1 <= keep <= groups or top > keep * (E // groups)):
         raise KernelError(f"routed_experts: {top} of {E} experts in {groups} groups of which {keep} are kept")
     if residual is None and not on_output:
@@ -1289,10 +1332,11 @@ def routed_experts(x: torch.Tensor, logits: torch.Tensor, w_gate: torch.Tensor, 
     place = empty((T * top,), torch.int32, dev)
     tile_expert = empty((cap // tile,), torch.int32, dev)
     y = empty((cap, F), x.dtype, dev)
-    _check(lib.st_moe_route(_ptr(ids), _ptr(wts), _ptr(logits), _ptr(token_item), T, E, int(top), mode, int(groups), int(keep), st))
+    _check(lib.st_moe_route(_ptr(ids), _ptr(wts), _ptr(logits), _ptr(token_item),
+                            _ptr(correction) if mode == 3 else None, float(scale), T, E, int(top), mode, int(groups), int(keep), st))
     _check(lib.st_moe_align(_ptr(sorted_pairs), _ptr(place), _ptr(tile_expert), _ptr(ids), T * top, E, cap, tile, st))
     _check(lib.st_moe_up(_ptr(y), _ptr(x), _ptr(w_gate), _ptr(w_up), _ptr(sorted_pairs), _ptr(tile_expert),
-                         _ptr(wts), cap, tile, int(top), W, F, float(limit), int(on_output), code, st))
+                         _ptr(wts), cap, tile, int(top), W, F, float(limit), 2 if w_gate is None else int(on_output), code, st))
     if on_output:
         out = residual if residual is not None else empty((T, W), torch.float32, dev)
         pair_out = empty((cap, W), torch.float32, dev)
@@ -1562,6 +1606,176 @@ def qk_norm_write(qk: torch.Tensor, gain_q: torch.Tensor, gain_k: torch.Tensor, 
                                    _ptr(gain_q), _ptr(gain_k), _ptr(token_item), _ptr(positions), _ptr(block_table),
                                    block_table.shape[1], ps, T, heads, kv_heads, head_dim, pad, float(eps), int(write),
                                    dtype_code(k_cache.dtype), _stream()))
+    return out
+
+
+# ------------------------------------------- root-mean-square norm in groups
+@_timed("group_rms", lambda x, gain, groups, eps, *, rows=None, out_t=None, out_f32=None: {
+    "rows": rows.shape[0] if rows is not None else x.shape[0], "width": x.shape[1],
+    "bytes": (rows.shape[0] if rows is not None else x.shape[0]) * x.shape[1] *
+             (4 + (out_t.element_size() if out_t is not None else 0) + 4 * (out_f32 is not None))})
+def group_rms(x: torch.Tensor, gain: torch.Tensor, groups: int, eps: float, *, rows: Optional[torch.Tensor] = None,
+              out_t: Optional[torch.Tensor] = None, out_f32: Optional[torch.Tensor] = None) -> None:
+    """Every one of the ``groups`` equal consecutive parts of a float row divided by sqrt(mean of its squares + eps),
+    the whole times ``gain`` (float [W]).  ``rows`` (int32): row r reads x[rows[r]], zeros where negative."""
+    T, W = x.shape
+    n = rows.shape[0] if rows is not None else T
+    _need(x, "x", torch.float32, (T, W))
+    _need(gain, "gain", torch.float32, (W,))
+    if groups < 1 or W % groups:
+        raise KernelError(f"{W} channels do not divide into {groups} groups")
+    if rows is not None:
+        _need(rows, "rows", torch.int32, (n,))
+    if out_t is None and out_f32 is None:
+        raise KernelError("group_rms needs a destination")
+    if out_t is not None:
+        _need(out_t, "out_t", None, (n, W))
+    if out_f32 is not None:
+        _need(out_f32, "out_f32", torch.float32, (n, W))
+    _check(_lib().st_group_rms(_ptr(out_t), _ptr(out_f32), _ptr(x), _ptr(rows), _ptr(gain), n, W, int(groups), float(eps),
+                               dtype_code(out_t.dtype) if out_t is not None else F32, _stream()))
+
+
+@_timed("group_norm_conv", lambda x, sides, groups, eps, ctx_arrays, out_dtype, all_single=False: {
+    "rows": x.shape[0], "width": x.shape[1], "sides": len(sides),
+    "bytes": x.numel() * (4 + len(sides) * torch.empty((), dtype=out_dtype).element_size())})
+def group_norm_conv(x: torch.Tensor, sides, groups: int, eps: float, ctx_arrays, out_dtype: torch.dtype,
+                    all_single: bool = False):
+    """For one or two ``sides`` = (gain [W], filter [taps, W], state [slots, taps - 1, W] or None with one tap), all
+    float, over the rows of a batch: n = the norm of ``group_rms`` with the side's gain, y[t] = n[t] + sum_j filter[j] *
+    n(position of t - taps + 1 + j); what lies before an item's first row is read from the side's state, which is
+    then moved on.  Returns the sides' results [T, W] in ``out_dtype``.  ``ctx_arrays``: the batch's (token_item,
+    item_len, item_tok_off, item_slot); ``all_single``: no item has more than one row."""
+    token_item, item_len, item_tok_off, item_slot = ctx_arrays
+    T, W = x.shape
+    if not 1 <= len(sides) <= 2:
+        raise KernelError(f"group_norm_conv: one or two sides, not {len(sides)}")
+    taps = sides[0][1].shape[0]
+    if groups < 1 or W % groups:
+        raise KernelError(f"{W} channels do not divide into {groups} groups")
+    _need(x, "x", torch.float32, (T, W))
+    _need(token_item, "token_item", torch.int32, (T,))
+    B = item_slot.shape[0]
+    for name, v in (("item_len", item_len), ("item_tok_off", item_tok_off), ("item_slot", item_slot)):
+        _need(v, name, torch.int32, (B,))
+    args, outs = [], []
+    for gain, w, state in sides:
+        _need(gain, "gain", torch.float32, (W,))
+        _need(w, "filter", torch.float32, (taps, W))
+        stride = _slot_rows(state, "state", (taps - 1) * W) if taps > 1 else 0
+        out = empty((T, W), out_dtype, x.device)
+        outs.append(out)
+        args += [_ptr(out), _ptr(gain), _ptr(w), _ptr(state) if taps > 1 else None, stride]
+    if len(sides) == 1:
+        args += [None, None, None, None, 0]
+    _check(_lib().st_group_norm_conv(*args, _ptr(x), _ptr(token_item), _ptr(item_len), _ptr(item_tok_off), _ptr(item_slot), T, B,
+                                     W, int(groups), taps, float(eps), int(bool(all_single)), dtype_code(out_dtype), _stream()))
+    return outs
+
+
+# ------------------- queries and keys turned and normalised a head, with the page write
+@_timed("unit_qk_write", lambda qkv, heads, kv_heads, key_dim, value_dim, eps, freq, factor, k_cache, *a, **k: {
+    "rows": qkv.shape[0], "width": qkv.shape[1],
+    "bytes": qkv.shape[0] * (4 * ((heads + kv_heads) * key_dim + kv_heads * value_dim) +
+                             k_cache.element_size() * k_cache.shape[3] * (heads + 2 * kv_heads))})
+def unit_qk_write(qkv: torch.Tensor, heads: int, kv_heads: int, key_dim: int, value_dim: int, eps: float,
+                  freq: Optional[torch.Tensor], factor: Optional[torch.Tensor], k_cache: torch.Tensor,
+                  v_cache: torch.Tensor, token_item: torch.Tensor, positions: torch.Tensor, block_table: torch.Tensor,
+                  write: bool = True) -> torch.Tensor:
+    """qkv: float rows (dense, any stride) that start with q [heads * key_dim] | k [kv_heads * key_dim] | v [kv_heads *
+    value_dim].  Of every query and key head the first 2 * len(freq) coordinates are turned by the row's position (i with
+    i + len(freq), angle position * freq[i]; ``freq`` None: none), then the head is divided by its root mean square (eps
+    inside the root); queries are multiplied by ``factor`` [heads] (None: 1).  Returns the queries [T, heads * pad] in
+    the pools' type (pad: the pools' entry width, zeros behind key_dim) and, with ``write``, stores keys and values
+    (as projected) in their pools [pages, kv_heads, page_size, pad]."""
+    num_pages, nkv, ps, pad = k_cache.shape
+    T = qkv.shape[0]
+    _need(qkv, "qkv", torch.float32, (T, qkv.shape[1]), contiguous=False)
+    if qkv.stride(1) != 1 or qkv.shape[1] < (heads + kv_heads) * key_dim + kv_heads * value_dim:
+        raise KernelError("qkv: dense rows that hold q, k and v")
+    if nkv != kv_heads or pad < max(key_dim, value_dim) or tuple(v_cache.shape) != tuple(k_cache.shape) or \
+            k_cache.stride()[1:] != (ps * pad, pad, 1) or v_cache.stride() != k_cache.stride():
+        raise KernelError("unit_qk_write: the pools do not fit the keys and values")
+    half = freq.shape[0] if freq is not None else 0
+    if freq is not None:
+        _need(freq, "freq", torch.float32, (half,))
+    if factor is not None:
+        _need(factor, "factor", torch.float32, (heads,))
+    _need(token_item, "token_item", torch.int32, (T,))
+    _need(positions, "positions", torch.int32, (T,))
+    _need(block_table, "block_table", torch.int32)
+    out = empty((T, heads * pad), k_cache.dtype, qkv.device)
+    _check(_lib().st_unit_qk_write(_ptr(out), _ptr(k_cache), _ptr(v_cache), k_cache.stride(0), _ptr(qkv), qkv.stride(0),
+                                   _ptr(freq), half, _ptr(factor), _ptr(token_item), _ptr(positions), _ptr(block_table),
+                                   block_table.shape[1], ps, T, heads, kv_heads, key_dim, value_dim, pad, float(eps),
+                                   int(write), dtype_code(k_cache.dtype), _stream()))
+    return out
+
+
+# ------------------------------------------- matrix memory with exponential gates
+def memory_row(heads: int, key_dim: int, value_dim: int) -> int:
+    """Floats of a row of ``matrix_memory``'s input: q | k | v | gate | log input gate | log forget gate."""
+    return 2 * heads * (key_dim + value_dim + 1)
+
+
+def memory_slot(heads: int, key_dim: int, value_dim: int) -> int:
+    """Floats of a request's state: S [heads, key_dim, value_dim] | n [heads, key_dim] | m [heads], filled up to whole
+    16-byte pieces."""
+    return -(-heads * (key_dim * value_dim + key_dim + 1) // 4) * 4
+
+
+def _d_memory(proj, bias_i, bias_f, gain, state, ctx_arrays, heads, key_dim, value_dim, cap, eps, out_dtype,
+              all_single=False):
+    T, B = proj.shape[0], ctx_arrays[3].shape[0]
+    es = torch.empty((), dtype=out_dtype).element_size()
+    return {"rows": T, "heads": heads, "key_dim": key_dim, "value_dim": value_dim, "items": B,
+            "flops": 6 * T * heads * key_dim * value_dim,
+            "bytes": T * (4 * memory_row(heads, key_dim, value_dim) + es * heads * value_dim) +
+                     8 * B * memory_slot(heads, key_dim, value_dim)}
+
+
+@_timed("matrix_memory", _d_memory)
+def matrix_memory(proj: torch.Tensor, bias_i: torch.Tensor, bias_f: torch.Tensor, gain: torch.Tensor, state: torch.Tensor,
+                  ctx_arrays, heads: int, key_dim: int, value_dim: int, cap: float, eps: float, out_dtype: torch.dtype,
+                  all_single: bool = False) -> torch.Tensor:
+    """Per item and head, from the slot's (S, n, m) and over the item's rows in order, with q scaled by key_dim^-1/2,
+    i = cap tanh((zi + bias_i) / cap) and f = log sigmoid(cap tanh((zf + bias_f) / cap)):
+    m' = max(f + m, i); S <- e^(f+m-m') S + e^(i-m') k v^T; n likewise with k; o = S^T q / (max(|n . q|, e^-m') + 1e-6);
+    the result is o at unit root mean square a head (eps inside the root), times ``gain`` [heads * value_dim], times
+    sigmoid(gate), in ``out_dtype``.  The state is stored back.
+
+    proj: float rows (dense, any stride) that start with q | k | v | gate | zi | zf (``memory_row``); state: float
+    [slots, memory_slot].  ``all_single``: every item has one row (one kernel); otherwise products within chunks of
+    rows and a carry between chunks.  Rows of no item are left as they are."""
+    _token_item, item_len, item_tok_off, item_slot = ctx_arrays
+    T = proj.shape[0]
+    if key_dim > 256 or value_dim > 256:
+        raise KernelError(f"matrix_memory: up to 256 key and value channels a head, not {key_dim} and {value_dim}")
+    _need(proj, "proj", torch.float32, (T, proj.shape[1]), contiguous=False)
+    if proj.stride(1) != 1 or proj.shape[1] < memory_row(heads, key_dim, value_dim):
+        raise KernelError("proj: dense rows that hold q, k, v, the gate and the log gates")
+    _need(bias_i, "bias_i", torch.float32, (heads,))
+    _need(bias_f, "bias_f", torch.float32, (heads,))
+    _need(gain, "gain", torch.float32, (heads * value_dim,))
+    slot_stride = _slot_rows(state, "state", memory_slot(heads, key_dim, value_dim))
+    B = item_slot.shape[0]
+    for name, t in (("item_len", item_len), ("item_tok_off", item_tok_off), ("item_slot", item_slot)):
+        _need(t, name, torch.int32, (B,))
+    lib, dev, code = _lib(), proj.device, dtype_code(out_dtype)
+    out = empty((T, heads * value_dim), out_dtype, dev)
+    q_scale = float(key_dim) ** -0.5
+    head = (_ptr(out), _ptr(proj), proj.stride(0), _ptr(state), slot_stride, _ptr(bias_i), _ptr(bias_f), _ptr(gain),
+            _ptr(item_len), _ptr(item_tok_off), _ptr(item_slot), B)
+    if all_single:
+        _check(lib.st_memory_step(*head, heads, key_dim, value_dim, float(cap), q_scale, float(eps), code, _stream()))
+        return out
+    chunks = T // int(lib.st_memory_chunk_rows()) + B
+    u = empty((chunks, heads, key_dim, value_dim), torch.float32, dev)
+    n = empty((chunks, heads, key_dim), torch.float32, dev)
+    sc = empty((chunks, heads, 2), torch.float64, dev)
+    m = empty((chunks, heads), torch.float32, dev)
+    _check(lib.st_memory_chunks(*head, T, heads, key_dim, value_dim, float(cap), q_scale, float(eps), _ptr(u), _ptr(n),
+                                _ptr(sc), _ptr(m), chunks, code, _stream()))
     return out
 
 

@@ -12,6 +12,9 @@ sandwich (norms before and after each sublayer; the reference has no such block)
 hyper-connections (several copies of the stream; the reference has no such block):
     u = sum_s a1[s] x_s;  y = Mix(N1(u));  x_t <- sum_s M1[s, t] x_s + b1[t] y   (all t at once)
     and the same with a2, M2, b2 around the feed-forward, which is optional
+parallel (both sublayers read the same stream; the reference has no such block):
+    x' = x + Mix(C1(N1(x))) + FFN(C2(N2(x)))
+    (C1 and C2 short filters over time; they and the feed-forward are optional)
 The residual stream is float; parts that multiply matrices take the storage type."""
 from __future__ import annotations
 
@@ -110,6 +113,57 @@ class Sandwich(Part):
         if side is not None:
             x32 = side.forward(x32, ctx, x_t=x_t)
         return x32
+
+
+class ParallelResidual(Part):
+    """params: feed_forward (bool, default True), taps (int: of a file's unused second filter).  A factor on the branches
+    is the mixer's and the feed-forward's own parameter.  The two norms and filters of a layer read the same rows: where
+    both are root-mean-square norms in equal groups behind filters of equal length (``GroupRmsNorm`` and
+    ``CausalTokenConv``), one kernel forms the statistics once and makes both inputs."""
+
+    def __init__(self, spec, hidden_size, dtype):
+        super().__init__(spec, hidden_size, dtype)
+        self.has_ffn = bool(spec.params.get("feed_forward", True))
+        self.taps = int(spec.params.get("taps", 0) or 0)
+        self.needs = ("mixer_norm", "ffn_norm", "feed_forward") if self.has_ffn else ("mixer_norm",)
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        # a layer without feed-forward: a file may still hold its norm and filter; they are not read
+        specs = []
+        if "unused_norm" in self.spec.names:
+            specs.append(TensorSpec(self.name("unused_norm"), (self.hidden_size,), "vector", optional=True))
+        if "unused_filter" in self.spec.names and self.taps:
+            specs.append(TensorSpec(self.name("unused_filter"), (self.hidden_size, self.taps), "vector", optional=True))
+        return specs
+
+    @staticmethod
+    def _fused(norm, conv) -> bool:
+        return (type(norm).__name__ == "GroupRmsNorm" and type(conv).__name__ == "CausalTokenConv" and conv.add_input)
+
+    def _inputs(self, x32, layer, ctx, conv_cache, ffn_conv_cache):
+        """What the mixer and the feed-forward (None without one) read, in the storage type."""
+        sides = [(layer.mixer_norm, layer.mixer_conv, conv_cache)]
+        if self.has_ffn:
+            sides.append((layer.ffn_norm, layer.ffn_conv, ffn_conv_cache))
+        first, conv = sides[0][0], sides[0][1]
+        if all(self._fused(n, c) and (n.groups, n.eps, c.taps) == (first.groups, first.eps, conv.taps) for n, c, _ in sides):
+            made = K.group_norm_conv(x32, [(n.gamma, c.weight_by_tap, cache.state) for n, c, cache in sides], first.groups,
+                                     first.eps, (ctx.token_item, ctx.item_len, ctx.item_tok_off, ctx.item_slot), self.dtype,
+                                     all_single=bool(ctx.all_single))
+        else:
+            made = []
+            for n, c, cache in sides:
+                if c is None:
+                    made.append(n.forward(x32, out_t=True)[0])
+                else:
+                    made.append(c.forward(n.forward(x32, out_t=False, out_f32=True)[1], ctx, cache))
+        return made[0], made[1] if self.has_ffn else None
+
+    def forward(self, x32: torch.Tensor, layer, ctx, cache, write: bool = True, conv_cache=None,
+                ffn_conv_cache=None) -> torch.Tensor:
+        a, d = self._inputs(x32, layer, ctx, conv_cache, ffn_conv_cache)
+        r32 = layer.mixer.forward(a, x32, ctx, cache, write)
+        return layer.feed_forward.forward(d, r32, ctx) if self.has_ffn else r32
 
 
 def _chains(norm, then) -> bool:

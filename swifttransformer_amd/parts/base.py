@@ -30,11 +30,11 @@ Kinds of part and their calls (x_t: activations in the engine's storage type
                 "state" need) and gets ``forward(ctx, position, cache=view)``
   head          ``forward(y_t) -> logits float32 [R, vocab]``
   arrangement   ``forward(x32, layer, ctx, cache, write) -> x32`` (with ``conv_cache=`` for a layer
-                that has a ``mixer_conv`` part); it may declare tensors of its own; ``reads_ahead`` True: it is
+                that has a ``mixer_conv`` part, and ``ffn_conv_cache=`` for one that has an ``ffn_conv``); it may declare tensors of its own; ``reads_ahead`` True: it is
                 called with ``then=`` the layer that runs next (or None) and may leave that layer's first input
                 in ``ctx.read_ahead``.  Where ``ModelSpec.streams`` is set, x32 is [T, streams * hidden]
   token_conv    ``cache_need() -> CacheNeed``; ``forward(y32, ctx, cache) -> y_t``: a short causal
-                filter over time on what a mixer reads, with its last inputs as per-request state
+                filter over time on what a mixer or a feed-forward reads, with its last inputs as per-request state
   side_input    ``forward(x32, ctx, x_t=None) -> x32`` (``x_t``: the stream in the storage type, if at hand): what a layer adds to the stream after its feed-forward
                 from an input of the token's own (a per-layer token embedding)
   reentry       ``forward(x32, first32, ctx) -> x32``: what happens to the residual stream before a run

@@ -43,12 +43,19 @@ register_part("mixer", "gated_window_attention", GatedWindowAttention)
 register_part("mixer", "retention", Retention)
 register_part("mixer", "parallel", ParallelMixers)
 register_part("side_input", "token_side", TokenSideInput)
-from .arrangement import HyperConnections
+from .arrangement import HyperConnections, ParallelResidual
 from .embedding import HashedPairEmbedding
 from .feed_forward import GatedFeedForward
+from .matrix_memory import MatrixMemory
+from .norm import GroupRmsNorm
 from .tied_attention import TiedKeyValueAttention
+from .unit_attention import UnitQueryKeyAttention
 
 register_part("arrangement", "hyper_connections", HyperConnections)
 register_part("embedding", "hashed_pairs", HashedPairEmbedding)
 register_part("feed_forward", "gated_dense", GatedFeedForward)
 register_part("mixer", "tied_kv_attention", TiedKeyValueAttention)
+register_part("arrangement", "parallel_residual", ParallelResidual)
+register_part("mixer", "matrix_memory", MatrixMemory)
+register_part("mixer", "unit_qk_attention", UnitQueryKeyAttention)
+register_part("norm", "group_rms", GroupRmsNorm)

@@ -28,13 +28,14 @@ class CausalTokenConv(Part):
         self.add_input = bool(spec.params.get("add_input", True))
         if not 1 <= self.taps <= 8:
             raise ValueError(f"the convolution kernel takes 1 to 8 taps, not {self.taps}")
-        self.weight = None
+        self.weight = self.weight_by_tap = None
 
     def tensor_specs(self) -> List[TensorSpec]:
         return [TensorSpec(self.name("weight"), (self.width, self.taps), "vector")]
 
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         self.weight = tensors[self.name("weight")]
+        self.weight_by_tap = self.weight.t().contiguous()      # [taps, width]: what the kernels fused with a norm read
 
     def cache_need(self) -> CacheNeed:
         return CacheNeed("state", state_shape=(self.taps - 1, self.width), state_dtype=torch.float32)

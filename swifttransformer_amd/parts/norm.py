@@ -11,7 +11,10 @@ the same kernels and the same fusion into a product, by a flag.
 ``DynamicTanh`` is a norm that takes no statistics of the row at all: y = tanh(alpha x) * w + b per
 element, alpha one learned number.  It can also add its result to a stream on the way
 (``forward_onto``), which is how a branch's result is normalised as it enters the residual stream.
-The reference has no such part."""
+The reference has no such part.
+
+``GroupRmsNorm`` divides every one of a row's equal consecutive parts by its own root mean square and multiplies the
+whole by a gain.  The reference has no such part."""
 from __future__ import annotations
 
 from typing import Dict, List, Optional, Tuple
@@ -128,3 +131,35 @@ class DynamicTanh(Part):
         K.dynamic_tanh(y32, self.gamma, self.beta, self.alpha, out_f32=out, out_t=out_t, base=stream32,
                        then=None if then is None else (then.gamma, then.beta, then.alpha))
         return out, out_t
+
+
+class GroupRmsNorm(Part):
+    """params: eps (float, inside the root), groups (int: equal consecutive parts of the row), width (int, default
+    hidden_size).  names: weight."""
+
+    def __init__(self, spec, hidden_size, dtype):
+        super().__init__(spec, hidden_size, dtype)
+        self.width = int(self.param("width", hidden_size))
+        self.eps = float(self.param("eps"))
+        self.groups = int(self.param("groups"))
+        if self.groups < 1 or self.width % self.groups:
+            raise ValueError(f"{self.width} channels do not divide into {self.groups} groups")
+        self.gamma: Optional[torch.Tensor] = None
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        return [TensorSpec(self.name("weight"), (self.width,), "vector", init="gain")]
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        self.gamma = tensors[self.name("weight")].contiguous()
+
+    def forward(self, x32: torch.Tensor, *, out_t: bool = True, out_f32: bool = False,
+                rows: Optional[torch.Tensor] = None) -> Tuple[Optional[torch.Tensor], Optional[torch.Tensor]]:
+        n = rows.shape[0] if rows is not None else x32.shape[0]
+        if self.dtype == torch.float32:                       # one float result serves as both
+            y = K.empty((n, self.width), torch.float32, x32.device)
+            K.group_rms(x32, self.gamma, self.groups, self.eps, rows=rows, out_f32=y)
+            return (y if out_t else None), (y if out_f32 else None)
+        yt = K.empty((n, self.width), self.dtype, x32.device) if out_t else None
+        y32 = K.empty((n, self.width), torch.float32, x32.device) if out_f32 else None
+        K.group_rms(x32, self.gamma, self.groups, self.eps, rows=rows, out_t=yt, out_f32=y32)
+        return yt, y32

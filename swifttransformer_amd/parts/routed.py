@@ -18,6 +18,13 @@ or, ``style`` "softmax_all":
     group ranks by its largest s, and the ``top`` largest s among the experts of the ``keep`` best groups choose
     the experts;  the token's result is sum_e s_e expert_e(x) with s as it is (not renormalised)
 
+or, ``style`` "sigmoid_output":
+
+    z = Wr x (float);  s = sigmoid(z);  the ``top`` largest s + correction choose the experts;  their weights are
+    scale * s_e / (the chosen s summed + 1e-20);  the token's result is sum_e weight_e expert_e(x)
+
+Experts without a gate (``gated`` False, not in the first style) are Wd gelu(Wu x), the exact GELU.
+
 Routing, sorting by expert and the experts' products all run on the device with launch shapes
 that depend on the number of rows only, so steps with this part are recorded like any other
 (``csrc/moe.hip``).  The reference has no such part."""
@@ -35,7 +42,8 @@ from .base import Part
 class RoutedExperts(Part):
     """params: experts (int), top (int), inner (int: width inside an expert), limit (float, of the
     "scaled_input" style), residual_scale (float, default 1), style ("scaled_input", the default, or
-    "softmax_output" or "softmax_all"), groups and keep (ints, default 1: of the "softmax_all" style),
+    "softmax_output", "softmax_all" or "sigmoid_output"), gated (bool, default True), scale (float, default 1: of the
+    "sigmoid_output" style, which also names a tensor ``correction`` [experts]), groups and keep (ints, default 1: of the "softmax_all" style),
     router_bias (bool, default False).  names: ``router`` (``router_bias``) and the
     patterns ``gate``, ``up``, ``down`` with ``{e}`` for the expert's number."""
 
@@ -55,6 +63,10 @@ class RoutedExperts(Part):
             raise ValueError(f"{self.experts} experts in {self.groups} equal groups (up to 64) of which {self.keep} are kept")
         if self.style == "softmax_all" and int(self.param("top")) > self.keep * (self.experts // self.groups):
             raise ValueError(f"{self.param('top')} experts a token do not fit {self.keep} groups")
+        self.gated = bool(spec.params.get("gated", True))
+        self.scale = float(spec.params.get("scale", 1.0))
+        if not self.gated and self.style == "scaled_input":
+            raise ValueError("experts without a gate go with weights on their results")
         self.residual_scale = float(spec.params.get("residual_scale", 1.0))
         if not 1 <= self.top <= min(self.experts, 16):
             raise ValueError(f"1 to 16 of {self.experts} experts a token, not {self.top}")
@@ -67,9 +79,12 @@ class RoutedExperts(Part):
         specs = [TensorSpec(self.name("router"), (self.experts, H), "matrix")]
         if self.router_bias:
             specs.append(TensorSpec(self.name("router_bias"), (self.experts,), "vector"))
+        if self.style == "sigmoid_output":
+            specs.append(TensorSpec(self.name("correction"), (self.experts,), "vector"))
         for e in range(self.experts):
-            specs += [TensorSpec(self._expert("gate", e), (F, H), "matrix"),
-                      TensorSpec(self._expert("up", e), (F, H), "matrix"),
+            if self.gated:
+                specs.append(TensorSpec(self._expert("gate", e), (F, H), "matrix"))
+            specs += [TensorSpec(self._expert("up", e), (F, H), "matrix"),
                       TensorSpec(self._expert("down", e), (H, F), "matrix")]
         return specs
 
@@ -77,10 +92,12 @@ class RoutedExperts(Part):
         self.w_router = tensors[self.name("router")]
         self.b_router = tensors[self.name("router_bias")] if self.router_bias else None
         stack = lambda which: torch.stack([tensors[self._expert(which, e)] for e in range(self.experts)]).contiguous()
-        self.w_gate, self.w_up, self.w_down = stack("gate"), stack("up"), stack("down")
+        self.w_gate = stack("gate") if self.gated else None
+        self.w_up, self.w_down = stack("up"), stack("down")
+        self.correction = tensors[self.name("correction")].contiguous() if self.style == "sigmoid_output" else None
 
     def forward(self, x_t: torch.Tensor, residual32: torch.Tensor, ctx) -> torch.Tensor:
         logits = K.gemm(x_t, self.w_router, bias=self.b_router, out_f32=True)
         return K.routed_experts(x_t, logits, self.w_gate, self.w_up, self.w_down, residual32, top=self.top,
                                 limit=self.limit, out_scale=self.residual_scale, token_item=ctx.token_item,
-                                style=self.style, groups=self.groups, keep=self.keep)
+                                style=self.style, groups=self.groups, keep=self.keep, correction=self.correction, scale=self.scale)
