@@ -145,7 +145,9 @@ class PlainFiterax:
         after = []
         for i, L in enumerate(cfg["layers"]):
             wm, wf, mlp = self.sub(f"l{i}.mix."), self.sub(f"l{i}.mlp."), L.get("mlp")
-            read = lambda which: input_conv(group_rms(x, t[f"l{i}.norm{which}"], groups, eps), t[f"l{i}.canon{which}"])
+            filtered = bool(cfg.get("canon"))
+            read = lambda which: (lambda n: input_conv(n, t[f"l{i}.canon{which}"]) if filtered else n)(
+                group_rms(x, t[f"l{i}.norm{which}"], groups, eps))
             mixer = {"attention": attention, "mlstm": mlstm}[L["type"]]
             y = mixer(read(1), wm, L["mixer"], eps)
             if mlp is not None:
