@@ -264,7 +264,7 @@ __global__ __launch_bounds__(256 * KS, HDP <= 2 ? 4 : 1) void attn_prefill_kerne
             for (int t = 0; t < 4; ++t)
 #pragma unroll
                 for (int r = 0; r < 4; ++r)
-                    st[t][r] = fmaf(cap_l2, tanhf(st[t][r] * inv_cap), bias_l2 * (float)(kb + 16 * t + 4 * g + r - qpos));
+                    st[t][r] = fmaf(cap_l2, tanh_fast(st[t][r] * inv_cap), bias_l2 * (float)(kb + 16 * t + 4 * g + r - qpos));
         } else if (biased) {
 #pragma unroll
             for (int t = 0; t < 4; ++t)

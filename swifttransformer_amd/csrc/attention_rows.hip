@@ -220,7 +220,7 @@ __global__ __launch_bounds__(512) void attn_rows_kernel(
 #pragma unroll
         for (int u = 0; u < U; ++u) {
             s[u] = fmaf(slope, (float)(j0 + u * G - pos), group_sum<LPK>(s[u]) * post_scale);   // slope 0: the score itself
-            if (softcap > 0.f) s[u] = softcap * tanhf(s[u] * inv_cap);
+            if (softcap > 0.f) s[u] = softcap * (ACC ? tanhf(s[u] * inv_cap) : tanh_fast(s[u] * inv_cap));
             if (j0 + u * G >= ke) s[u] = -INFINITY;      // the same for all lanes of a group
             mn = fmaxf(mn, s[u]);
         }

@@ -133,6 +133,12 @@ __device__ inline float rows4_sum(float x) {
     return __uint_as_float(b[0]) + __uint_as_float(b[1]);
 }
 
+// tanh as 1 - 2 / (1 + 2^(2 log2(e) x)) by the hardware's exponential and reciprocal: off by a few 2^-24 of one
+// (absolute), for scores that meet values of the 16-bit storage type
+__device__ inline float tanh_fast(float x) {
+    return fmaf(-2.f, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(2.88539008177792681f * x)), 1.f);
+}
+
 __device__ inline float wave_sum(float v) {
 #pragma unroll
     for (int o = kWave / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, kWave);

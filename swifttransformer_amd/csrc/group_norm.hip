@@ -95,26 +95,40 @@ struct NormConvSide {
     void* out;
 };
 
-// LDS: statistics [rows + taps - 1][groups], entry i of them belonging to batch row t0 - (taps - 1) + i.  V columns a
-// thread and turn (4: 16-byte accesses; groups, width and addresses allow them).  TAPS: 1 to 4, or 8 for any number
-// up to that.  Everything a thread's first row needs is asked for before the statistics are formed, so that a step
-// of few rows waits for one trip to memory.
-template <typename T, int SIDES, int V, int TAPS>
+// LDS: statistics [R + TAPS - 1][groups], entry i of them belonging to batch row t0 - (TAPS - 1) + i.  V columns a
+// thread and turn (4: 16-byte accesses; groups, width and addresses allow them), R rows a workgroup.  TAPS: 1 to 4, or
+// 8 for any number up to that.  What a thread needs (its columns of all the rows, gains, filters, for single tokens
+// the state) is asked for before the statistics are formed: few trips to memory, side by side.
+template <typename T, int SIDES, int V, int TAPS, int R>
 __global__ __launch_bounds__(512) void group_norm_conv_kernel(
     NormConvSide s0, NormConvSide s1, const float* __restrict__ x, const int* __restrict__ token_item,
     const int* __restrict__ item_len, const int* __restrict__ item_tok_off, const int* __restrict__ item_slot,
-    int num_tokens, int width, int groups, int num_taps, int rows, float eps) {
+    int num_tokens, int width, int groups, int num_taps, float eps) {
     extern __shared__ float nc_stat[];
-    const int hist = (TAPS < kNormMaxTaps ? TAPS : num_taps) - 1, part = width / groups;
-    const int t0 = blockIdx.x * rows;
-    const int n = min(rows, num_tokens - t0);
+    constexpr int HIST = TAPS - 1;                // rows before the workgroup's own that are kept at hand
+    const int hist = TAPS < kNormMaxTaps ? HIST : num_taps - 1, part = width / groups;
+    const int t0 = blockIdx.x * R;
+    const int n = min(R, num_tokens - t0);
     const NormConvSide side[2] = {s0, s1};
+    int slot[R], row[R];                          // slot of the row's request (-1: a padding row), row within its portion
+    bool single[R];
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+        const int item = i < n ? token_item[t0 + i] : -1;
+        slot[i] = item >= 0 ? item_slot[item] : -1;
+        row[i] = slot[i] >= 0 ? t0 + i - item_tok_off[item] : 0;
+        single[i] = slot[i] >= 0 && item_len[item] == 1;
+    }
     bool have_stats = false;
     for (int c = threadIdx.x * V; c < width || !have_stats; c += blockDim.x * V) {
         const bool live = c < width;
         const int cc = live ? c : 0;              // (a thread without columns still helps with the statistics)
         const int g = cc / part;
-        float gain[SIDES][V], w[SIDES][TAPS][V];
+        float gain[SIDES][V], w[SIDES][TAPS][V], xv[R + HIST][V], old[SIDES][TAPS][V];
+        // (rows before the batch or past it: a stand-in that is not used)
+#pragma unroll
+        for (int k = 0; k < R + HIST; ++k)
+            load_columns<V>(x + (int64_t)min(max(t0 - HIST + k, 0), num_tokens - 1) * width + cc, xv[k]);
 #pragma unroll
         for (int s = 0; s < SIDES; ++s) {
             load_columns<V>(side[s].gain + cc, gain[s]);
@@ -122,65 +136,89 @@ __global__ __launch_bounds__(512) void group_norm_conv_kernel(
             for (int b = 0; b < TAPS; ++b)        // [rows back]
                 load_columns<V>(side[s].w + (int64_t)max(hist - b, 0) * width + cc, w[s][b]);
         }
-        for (int i = 0; i < n; ++i) {
-            const int t = t0 + i;
-            const int item = token_item[t];
-            const int slot = item >= 0 ? item_slot[item] : -1;
-            const int r = slot >= 0 ? t - item_tok_off[item] : 0;     // row within the item's portion
-            const bool single = slot >= 0 && item_len[item] == 1;
-            // the row and the rows of this step that its filter reaches (others: a stand-in that is not used)
-            float xv[TAPS][V], old[SIDES][TAPS][V];
+        auto load_old = [&](int i) {
 #pragma unroll
-            for (int b = 0; b < TAPS; ++b)
-                load_columns<V>(x + (int64_t)(b <= hist && b <= r ? t - b : t) * width + cc, xv[b]);
-            if (slot >= 0 && r < hist) {
+            for (int s = 0; s < SIDES; ++s)
 #pragma unroll
-                for (int s = 0; s < SIDES; ++s)
+                for (int b = 1; b < TAPS; ++b)
+                    load_columns<V>(side[s].state + (int64_t)slot[i] * side[s].slot_stride +
+                                    (int64_t)min(max(hist + row[i] - b, 0), hist - 1) * width + cc, old[s][b]);
+        };
+        if (R == 1 && slot[0] >= 0 && row[0] < hist) load_old(0);
+        if (!have_stats) {                        // uniform over the workgroup
+            // the rows before the workgroup's own that its filters reach: back to where the first row's item starts
+            const int before = slot[0] >= 0 ? min(hist, row[0]) : 0;
+            const int units = (n + before) * groups, waves = blockDim.x >> 6, lane = threadIdx.x & 63;
+            const float* first = x + (int64_t)(t0 - before) * width;
+            float* stat = nc_stat + (HIST - before) * groups;
+            // (rows side by side in memory: unit u is the part that starts u * part floats behind the first row)
+            for (int u = threadIdx.x >> 6; u < units; u += 4 * waves) {
+                float ss[4];
+                if (part <= 64 * V) {             // a wave covers a part at once: four parts on their way
 #pragma unroll
-                    for (int b = 1; b < TAPS; ++b)
-                        load_columns<V>(side[s].state + (int64_t)slot * side[s].slot_stride +
-                                        (int64_t)min(max(hist + r - b, 0), hist - 1) * width + cc, old[s][b]);
-            }
-            if (!have_stats) {                    // uniform over the workgroup
-                // the rows before the workgroup's own that its filters reach: back to where the first row's item starts
-                const int before = slot >= 0 ? min(hist, r) : 0;
-                const int waves = blockDim.x >> 6;
-                for (int u = threadIdx.x >> 6; u < (n + before) * groups; u += waves) {
-                    const int q = u / groups, gg = u - q * groups;
-                    const float rstd = group_rstd(x + (int64_t)(t0 - before + q) * width + gg * part, part, eps, V == 4);
-                    if ((threadIdx.x & 63) == 0) nc_stat[(hist - before + q) * groups + gg] = rstd;
+                    for (int j = 0; j < 4; ++j) {
+                        float v[V];
+                        const int at = lane * V;
+                        load_columns<V>(first + (int64_t)min(u + j * waves, units - 1) * part + min(at, part - V), v);
+                        ss[j] = 0.f;
+#pragma unroll
+                        for (int e = 0; e < V; ++e) ss[j] = at < part ? fmaf(v[e], v[e], ss[j]) : ss[j];
+                    }
+                } else {
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) ss[j] = 0.f;
+                    for (int at = lane * V; at < part; at += 64 * V) {
+#pragma unroll
+                        for (int j = 0; j < 4; ++j) {
+                            float v[V];
+                            load_columns<V>(first + (int64_t)min(u + j * waves, units - 1) * part + at, v);
+#pragma unroll
+                            for (int e = 0; e < V; ++e) ss[j] = fmaf(v[e], v[e], ss[j]);
+                        }
+                    }
                 }
-                __syncthreads();
-                have_stats = true;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    ss[j] = wave_sum(ss[j]);
+                    if (lane == 0 && u + j * waves < units) stat[u + j * waves] = 1.f / sqrtf(ss[j] / (float)part + eps);
+                }
             }
-            if (!live) break;
-            if (slot < 0) {                       // a padding row of a batch of fixed size
+            __syncthreads();
+            have_stats = true;
+        }
+        if (!live) break;
+#pragma unroll
+        for (int k = 0; k < R + HIST; ++k) {
+            const float rstd = nc_stat[k * groups + g];      // (entries of rows that no filter here reaches: never used)
+#pragma unroll
+            for (int v = 0; v < V; ++v) xv[k][v] *= rstd;
+        }
+#pragma unroll
+        for (int i = 0; i < R; ++i) {
+            if (i >= n) break;
+            const int64_t t = t0 + i;
+            if (slot[i] < 0) {                    // a padding row of a batch of fixed size
                 const float zero[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                for (int s = 0; s < SIDES; ++s) store_columns<V>((T*)side[s].out + (int64_t)t * width + cc, zero);
+                for (int s = 0; s < SIDES; ++s) store_columns<V>((T*)side[s].out + t * width + cc, zero);
                 continue;
             }
-#pragma unroll
-            for (int b = 0; b < TAPS; ++b) {
-                const float rstd = nc_stat[(b <= hist && b <= r ? hist + i - b : hist + i) * groups + g];
-#pragma unroll
-                for (int v = 0; v < V; ++v) xv[b][v] *= rstd;
-            }
+            if (R > 1 && row[i] < hist) load_old(i);
 #pragma unroll
             for (int s = 0; s < SIDES; ++s) {
                 float own[V], acc[V];
 #pragma unroll
-                for (int v = 0; v < V; ++v) acc[v] = own[v] = xv[0][v] * gain[s][v];
+                for (int v = 0; v < V; ++v) acc[v] = own[v] = xv[HIST + i][v] * gain[s][v];
 #pragma unroll
                 for (int b = TAPS - 1; b >= 0; --b) {
                     if (b > hist) continue;
 #pragma unroll
                     for (int v = 0; v < V; ++v)
-                        acc[v] = fmaf(w[s][b][v], b <= r ? xv[b][v] * gain[s][v] : old[s][b][v], acc[v]);
+                        acc[v] = fmaf(w[s][b][v], b <= row[i] ? xv[HIST + i - b][v] * gain[s][v] : old[s][b][v], acc[v]);
                 }
-                store_columns<V>((T*)side[s].out + (int64_t)t * width + cc, acc);
-                if (single) {                      // r is 0: what lies b rows back was read from the state above
-                    float* st = side[s].state + (int64_t)slot * side[s].slot_stride + cc;
+                store_columns<V>((T*)side[s].out + t * width + cc, acc);
+                if (single[i]) {                  // its row is 0: what lies b rows back was read from the state above
+                    float* st = side[s].state + (int64_t)slot[i] * side[s].slot_stride + cc;
 #pragma unroll
                     for (int b = 1; b < TAPS; ++b) {
                         if (b > hist) continue;
@@ -193,45 +231,51 @@ __global__ __launch_bounds__(512) void group_norm_conv_kernel(
 }
 
 // a workgroup an item of several rows: the state becomes the last taps - 1 of (old state, the item's normed rows)
-template <int SIDES>
-__global__ __launch_bounds__(256) void group_norm_conv_state_kernel(
+template <int SIDES, int V>
+__global__ __launch_bounds__(512) void group_norm_conv_state_kernel(
     NormConvSide s0, NormConvSide s1, const float* __restrict__ x, const int* __restrict__ item_len,
-    const int* __restrict__ item_tok_off, const int* __restrict__ item_slot, int width, int groups, int taps, float eps,
-    int vec) {
+    const int* __restrict__ item_tok_off, const int* __restrict__ item_slot, int width, int groups, int taps, float eps) {
     extern __shared__ float nc_stat[];
     const int item = blockIdx.x;
     const int slot = item_slot[item], n = item_len[item];
     if (slot < 0 || n <= 1) return;
     const int hist = taps - 1, part = width / groups;
-    const float* xi = x + (int64_t)item_tok_off[item] * width;
-    const int wave = threadIdx.x >> 6;
-    for (int u = wave; u < hist * groups; u += 4) {
-        const int i = u / groups, g = u - i * groups;
-        const int p = n - hist + i;
-        if (p < 0) continue;
-        const float rstd = group_rstd(xi + (int64_t)p * width + g * part, part, eps, vec);
-        if ((threadIdx.x & 63) == 0) nc_stat[i * groups + g] = rstd;
+    const int fresh = min(n, hist), kept = hist - fresh;     // rows from this step, rows that move up in the state
+    const float* xi = x + (int64_t)(item_tok_off[item] + n - fresh) * width;
+    // (every workgroup of an item forms the statistics of all parts of the rows)
+    for (int u = threadIdx.x >> 6; u < fresh * groups; u += blockDim.x >> 6) {
+        const float rstd = group_rstd(xi + (int64_t)u * part, part, eps, V == 4);
+        if ((threadIdx.x & 63) == 0) nc_stat[u] = rstd;
+    }
+    const NormConvSide side[2] = {s0, s1};
+    const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
+    const bool live = c < width;
+    const int cc = live ? c : 0, g = cc / part;
+    float keep[SIDES][kNormMaxTaps][V], gain[SIDES][V];
+#pragma unroll
+    for (int s = 0; s < SIDES; ++s) {
+        const float* st = side[s].state + (int64_t)slot * side[s].slot_stride + cc;
+        load_columns<V>(side[s].gain + cc, gain[s]);
+#pragma unroll
+        for (int i = 0; i < kNormMaxTaps - 1; ++i) {
+            if (i >= hist) continue;
+            load_columns<V>(i < kept ? st + (int64_t)(i + fresh) * width : xi + (int64_t)(i - kept) * width + cc, keep[s][i]);
+        }
     }
     __syncthreads();
-    const NormConvSide* side[2] = {&s0, &s1};
-    for (int c = threadIdx.x; c < width; c += 256) {
-        const int g = c / part;
+    if (!live) return;
 #pragma unroll
-        for (int s = 0; s < SIDES; ++s) {
-            float* st = side[s]->state + (int64_t)slot * side[s]->slot_stride + c;
-            const float gain = side[s]->gain[c];
-            float keep[kNormMaxTaps];
+    for (int s = 0; s < SIDES; ++s) {
+        float* st = side[s].state + (int64_t)slot * side[s].slot_stride + cc;
 #pragma unroll
-            for (int i = 0; i < kNormMaxTaps; ++i) {
-                if (i >= hist) continue;
-                const int p = n - hist + i;         // row of the portion, negative: still in the old state
-                keep[i] = p >= 0 ? xi[(int64_t)p * width + c] * nc_stat[i * groups + g] * gain : st[(int64_t)(hist + p) * width];
+        for (int i = 0; i < kNormMaxTaps - 1; ++i) {
+            if (i >= hist) continue;
+            if (i >= kept) {
+                const float rstd = nc_stat[(i - kept) * groups + g];
+#pragma unroll
+                for (int v = 0; v < V; ++v) keep[s][i][v] *= rstd * gain[s][v];
             }
-#pragma unroll
-            for (int i = 0; i < kNormMaxTaps; ++i) {
-                if (i >= hist) continue;
-                st[(int64_t)i * width] = keep[i];
-            }
+            store_columns<V>(st + (int64_t)i * width, keep[s][i]);
         }
     }
 }
@@ -285,15 +329,20 @@ extern "C" int st_group_norm_conv(void* out0, const float* gain0, const float* w
     ST_CHECK(!out1 || (gain1 && w1 && (state1 || taps == 1)), "group_norm_conv: null operand of the second side");
     const NormConvSide a{gain0, w0, state0, slot_stride0, out0}, b{gain1, w1, state1, slot_stride1, out1};
     // several rows a workgroup only where that leaves enough workgroups to fill the chip
-    const int rows = num_tokens >= kNormRows * device_compute_units() ? kNormRows : 1;
+    // (and where the registers hold several rows' window of a filter)
+    const bool many = taps <= 4 && num_tokens >= kNormRows * device_compute_units();
+    const int rows = many ? kNormRows : 1;
     const bool vec = (width / groups) % 4 == 0 && aligned16(x, out0, gain0, w0) && aligned16(out1, gain1, w1) &&
                      aligned16(state0, state1) && slot_stride0 % 4 == 0 && slot_stride1 % 4 == 0;
     const unsigned grid = (unsigned)((num_tokens + rows - 1) / rows);
-    const int threads = rows == 1 && width > 256 * (vec ? 4 : 1) ? 512 : 256;
-    const size_t lds = sizeof(float) * (size_t)(rows + taps - 1) * groups;
-#define ST_NC(T, S, V, K)                                                                                             \
-    group_norm_conv_kernel<T, S, V, K><<<grid, threads, lds, stream>>>(a, b, x, token_item, item_len, item_tok_off,    \
-                                                                      item_slot, num_tokens, width, groups, taps, rows, eps)
+    const int threads = width > 256 * (vec ? 4 : 1) ? 512 : 256;
+    const int kept_taps = taps <= 4 ? taps : kNormMaxTaps;
+    const size_t lds = sizeof(float) * (size_t)(rows + kept_taps - 1) * groups;
+#define ST_NC(T, S, V, K) do {                                                                                        \
+        if (many) group_norm_conv_kernel<T, S, V, (K <= 4 ? K : 4), kNormRows><<<grid, threads, lds, stream>>>(a, b, x, token_item,   \
+            item_len, item_tok_off, item_slot, num_tokens, width, groups, taps, eps);                                  \
+        else group_norm_conv_kernel<T, S, V, K, 1><<<grid, threads, lds, stream>>>(a, b, x, token_item, item_len,      \
+            item_tok_off, item_slot, num_tokens, width, groups, taps, eps); } while (0)
 #define ST_NC_K(T, S, V) do { switch (taps) { case 1: ST_NC(T, S, V, 1); break; case 2: ST_NC(T, S, V, 2); break;    \
         case 3: ST_NC(T, S, V, 3); break; case 4: ST_NC(T, S, V, 4); break; default: ST_NC(T, S, V, 8); } } while (0)
 #define ST_NC_T(T) do { if (out1) { if (vec) ST_NC_K(T, 2, 4); else ST_NC_K(T, 2, 1); }                              \
@@ -305,12 +354,15 @@ extern "C" int st_group_norm_conv(void* out0, const float* gain0, const float* w
     ST_LAUNCH_CHECK("group_norm_conv");
     if (all_single || taps == 1 || num_items == 0) return 0;
     const size_t lds2 = sizeof(float) * (size_t)(taps - 1) * groups;
-    if (out1)
-        group_norm_conv_state_kernel<2><<<num_items, 256, lds2, stream>>>(a, b, x, item_len, item_tok_off, item_slot, width,
-                                                                          groups, taps, eps, vec);
-    else
-        group_norm_conv_state_kernel<1><<<num_items, 256, lds2, stream>>>(a, b, x, item_len, item_tok_off, item_slot, width,
-                                                                          groups, taps, eps, vec);
+    const int per = 512 * (vec ? 4 : 1);
+    ST_CHECK((width + per - 1) / per <= 65535, "group_norm_conv: rows too wide");
+    // (a workgroup writes its own columns of the state only, and has read them before)
+    const dim3 grid2(num_items, (width + per - 1) / per);
+#define ST_NS(S, V) group_norm_conv_state_kernel<S, V><<<grid2, 512, lds2, stream>>>(a, b, x, item_len, item_tok_off, item_slot, \
+                                                                                   width, groups, taps, eps)
+    if (out1) { if (vec) ST_NS(2, 4); else ST_NS(2, 1); }
+    else { if (vec) ST_NS(1, 4); else ST_NS(1, 1); }
+#undef ST_NS
     ST_LAUNCH_CHECK("group_norm_conv (state)");
     return 0;
 }

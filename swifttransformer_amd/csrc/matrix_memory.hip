@@ -24,6 +24,9 @@
 #include "api.h"
 #include "common.h"
 
+#include <mutex>
+#include <set>
+
 namespace st {
 
 typedef float floatx4 __attribute__((ext_vector_type(4)));
@@ -203,10 +206,63 @@ __device__ inline double wave_max_double(double v) {
     return v;
 }
 
+// Four neighbouring floats of a row, zeros past its `limit` numbers or where the row does not exist.  VEC: the row starts
+// on 16 bytes and the limit is a multiple of 4.  (Addresses are clamped and values cleared rather than loads behind a
+// branch: the loads of a tile are then all on their way at once.)
+template <bool VEC>
+__device__ inline float4 load_piece(const float* __restrict__ row, int c, int limit, bool ok) {
+    float4 v;
+    if (VEC) {
+        v = *reinterpret_cast<const float4*>(row + min(c, limit - 4));
+    } else {
+        v.x = row[min(c, limit - 1)];
+        v.y = row[min(c + 1, limit - 1)];
+        v.z = row[min(c + 2, limit - 1)];
+        v.w = row[min(c + 3, limit - 1)];
+    }
+    v.x = ok && c < limit ? v.x : 0.f;
+    v.y = ok && c + 1 < limit ? v.y : 0.f;
+    v.z = ok && c + 2 < limit ? v.z : 0.f;
+    v.w = ok && c + 3 < limit ? v.w : 0.f;
+    return v;
+}
+
+// A tile of 64 rows x 4 * P4 floats (P4 a power of two) by 256 threads: piece i of a thread is row e / P4, floats 4 (e % P4)
+// on, e = thread + 256 i; P4 / 4 pieces a thread.
+template <int P4>
+struct Tile {
+    static constexpr int kPieces = P4 / 4;
+    float4 v[kPieces];
+    template <bool VEC>
+    __device__ inline void load(const float* __restrict__ base, int64_t stride, int rows, int first, int limit) {
+#pragma unroll
+        for (int i = 0; i < kPieces; ++i) {
+            const int e = threadIdx.x + 256 * i, j = e / P4, c = 4 * (e % P4);
+            v[i] = load_piece<VEC>(base + (int64_t)min(j, rows - 1) * stride, first + c, limit, j < rows);
+        }
+    }
+    __device__ inline void store(float* lds, int lds_stride) const {
+#pragma unroll
+        for (int i = 0; i < kPieces; ++i) {
+            const int e = threadIdx.x + 256 * i;
+            *reinterpret_cast<float4*>(lds + (e / P4) * lds_stride + 4 * (e % P4)) = v[i];
+        }
+    }
+    __device__ inline void store_weighted(float* lds, int lds_stride, const float* w) const {
+#pragma unroll
+        for (int i = 0; i < kPieces; ++i) {
+            const int e = threadIdx.x + 256 * i;
+            const float f = w[e / P4];
+            *reinterpret_cast<float4*>(lds + (e / P4) * lds_stride + 4 * (e % P4)) = make_float4(v[i].x * f, v[i].y * f, v[i].z * f, v[i].w * f);
+        }
+    }
+};
+
 // U[idx, head] = sum_j e^(c_j - max c) k_j v_j^T [dk, dv], N[idx, head] the same sum of k_j, scal[idx, head] =
-// (F of the whole chunk, max c).  Grid (heads, chunks, blocks of 64 value channels); a wave takes 16 x 16 tiles.
-// LDS: k [64][dk16 + 4] (weighted), v [64][68], weights [64].  A matrix instruction sums 4 keys: lane group g of tile
-// step s takes key 16 (s / 4) + 4 g + s % 4, which spreads its reads over the banks.
+// (F of the whole chunk, max c).  Grid (heads, chunks, blocks of 64 value channels); a wave takes rows of 16 x 16 tiles.
+// KQ: dk <= 4 KQ.  LDS: k [64][4 KQ + 4] (weighted), v [64][68], weights [64].  A matrix instruction sums 4 keys: lane
+// group g of step (s, r) takes key 16 s + 4 g + r, which spreads its reads over the banks.
+template <int KQ, bool VEC>
 __global__ __launch_bounds__(256) void memory_sums_kernel(
     float* __restrict__ U, float* __restrict__ N, double* __restrict__ scal, const float* __restrict__ proj, int64_t stride,
     const float* __restrict__ bias_i, const float* __restrict__ bias_f, const int* __restrict__ item_len,
@@ -218,11 +274,15 @@ __global__ __launch_bounds__(256) void memory_sums_kernel(
     const int n = min(kMemChunk, item_len[item] - chunk * kMemChunk);
     const int64_t row0 = (int64_t)item_tok_off[item] + (int64_t)chunk * kMemChunk;
     const float* p = proj + row0 * stride;
-    const int dk = sh.dk, dv = sh.dv, ktiles = (dk + 15) >> 4, KS = 16 * ktiles + 4;
-    constexpr int VS = 68;
+    const int dk = sh.dk, dv = sh.dv, ktiles = (dk + 15) >> 4;
+    constexpr int KS = 4 * KQ + 4, VS = 68;
     float* ks = mem_lds;
     float* vs = ks + kMemChunk * KS;
     float* w = vs + kMemChunk * VS;
+    Tile<KQ> tk;
+    Tile<16> tv;
+    tk.template load<VEC>(p + sh.k_off() + (int64_t)head * dk, stride, n, 0, dk);
+    tv.template load<VEC>(p + sh.v_off() + (int64_t)head * dv, stride, n, vb, dv);
     if (tid < 64) {
         double F, c, last;
         memory_chunk_gates(F, c, last, p, stride, bias_i, bias_f, sh, head, n, cap);
@@ -233,29 +293,16 @@ __global__ __launch_bounds__(256) void memory_sums_kernel(
             scal[((int64_t)idx * sh.heads + head) * 2 + 1] = mx;
         }
     }
-    for (int e = tid; e < kMemChunk * 64; e += 256) {
-        const int j = e >> 6, col = vb + (e & 63);
-        vs[j * VS + (e & 63)] = (j < n && col < dv) ? p[(int64_t)j * stride + sh.v_off() + (int64_t)head * dv + col] : 0.f;
-    }
+    tv.store(vs, VS);
     __syncthreads();                                // the weights
-    const int kw = 16 * ktiles;
-    for (int e = tid; e < kMemChunk * kw; e += 256) {
-        const int j = e / kw, kk = e - j * kw;
-        ks[j * KS + kk] = (j < n && kk < dk) ? p[(int64_t)j * stride + sh.k_off() + (int64_t)head * dk + kk] * w[j] : 0.f;
-    }
+    tk.store_weighted(ks, KS, w);
     __syncthreads();
-    if (blockIdx.z == 0) {
-        for (int kk = tid; kk < dk; kk += 256) {
-            float sum = 0.f;
-            for (int j = 0; j < n; ++j) sum += ks[j * KS + kk];
-            N[((int64_t)idx * sh.heads + head) * dk + kk] = sum;
-        }
-    }
     const int lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
     const int steps = (n + 15) >> 4;                // 16 keys each
     float* u = U + ((int64_t)idx * sh.heads + head) * dk * dv;
+    const bool with_n = blockIdx.z == 0;
     for (int kt = wave; kt < ktiles; kt += 4) {
-        floatx4 acc[4];
+        floatx4 acc[4], an = floatx4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int vt = 0; vt < 4; ++vt) acc[vt] = floatx4{0.f, 0.f, 0.f, 0.f};
         for (int s = 0; s < steps; ++s) {
@@ -263,6 +310,7 @@ __global__ __launch_bounds__(256) void memory_sums_kernel(
             for (int r = 0; r < 4; ++r) {
                 const int j = 16 * s + 4 * g + r;
                 const float a = ks[j * KS + 16 * kt + r16];
+                if (with_n) an = __builtin_amdgcn_mfma_f32_16x16x4f32(a, 1.f, an, 0, 0, 0);
 #pragma unroll
                 for (int vt = 0; vt < 4; ++vt)
                     acc[vt] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, vs[j * VS + 16 * vt + r16], acc[vt], 0, 0, 0);
@@ -270,13 +318,14 @@ __global__ __launch_bounds__(256) void memory_sums_kernel(
         }
         // acc[vt][r]: key channel 16 kt + 4 g + r, value channel 16 vt + r16
 #pragma unroll
-        for (int vt = 0; vt < 4; ++vt) {
-            const int col = vb + 16 * vt + r16;
-            if (col >= dv) continue;
+        for (int r = 0; r < 4; ++r) {
+            const int kk = 16 * kt + 4 * g + r;
+            if (kk >= dk) continue;
+            if (with_n && r16 == 0) N[((int64_t)idx * sh.heads + head) * dk + kk] = an[r];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int kk = 16 * kt + 4 * g + r;
-                if (kk < dk) u[(int64_t)kk * dv + col] = acc[vt][r];
+            for (int vt = 0; vt < 4; ++vt) {
+                const int col = vb + 16 * vt + r16;
+                if (col < dv) u[(int64_t)kk * dv + col] = acc[vt][r];
             }
         }
     }
@@ -308,7 +357,7 @@ __global__ __launch_bounds__(256) void memory_carry_kernel(
     const double* sc = scal + first * 2;
     float S = *home;
     double m = (double)sl[sh.m_base() + head];
-    constexpr int B = 8;                            // chunks asked for at once
+    constexpr int B = 16;                           // chunks asked for at once
     for (int c0 = 0; c0 < chunks; c0 += B) {
         float add[B];
         double total[B], mx[B];
@@ -334,17 +383,27 @@ __global__ __launch_bounds__(256) void memory_carry_kernel(
 
 // Rows of a chunk, transposed: S^T = K Q^T leaves a lane with keys 4 g + r of ONE row (lane % 16), so weights, the
 // denominator and the norm are per-lane numbers and sums over the four lane groups, and the weighted scores are the
-// next product's operand as they lie (O^T += V^T P^T, 4 keys an instruction: key 4 g + r of lane group g).
-// Four waves, 16 rows each.  NV: tiles of 16 value channels (dv <= 16 NV); KQ: key channels a lane group (dk <= 4 KQ).
-// LDS: k [64][4 KQ + 4] | v [64][68] (a block of 64 value channels at a time) | c, M doubles [64] each.
-template <typename T, int KQ, int NV>
+// next product's operand as they lie (O^T += V^T P^T, 4 keys an instruction: key 4 g + r of lane group g).  Key channel
+// 4 s + g belongs to lane group g in step s of the products over key channels.
+// Four waves, 16 rows each.  NV: tiles of 16 value channels (dv <= 16 NV); KQ: dk <= 4 KQ.
+// LDS: c, M doubles [64] each | m [64] | k [64][4 KQ + 4], later 64 key channels of the start state [64][16 NV + 16] |
+// v [64][16 NV + 4]: strides that spread the instructions' reads over the banks.
+template <int KQ, int NV>
+struct MemoryOutLds {
+    static constexpr int KS = 4 * KQ + 4, VS = 16 * NV + 4, SS = 16 * NV + 16;
+    static constexpr int first = KS > SS ? 64 * KS : 64 * SS;
+    static constexpr size_t bytes = sizeof(double) * 2 * kMemChunk + sizeof(float) * (size_t)(kMemChunk + first + 64 * VS);
+};
+
+template <typename T, int KQ, int NV, bool VEC>
 __global__ __launch_bounds__(256) void memory_out_kernel(
     T* __restrict__ out, const float* __restrict__ proj, int64_t stride, float* __restrict__ state, int64_t slot_stride,
-    const float* __restrict__ S0, const float* __restrict__ N0, const float* __restrict__ start_m, const float* __restrict__ bias_i,
-    const float* __restrict__ bias_f, const float* __restrict__ gain, const int* __restrict__ item_len,
-    const int* __restrict__ item_tok_off, const int* __restrict__ item_slot, int num_items, MemoryShape sh, float cap,
-    float q_scale, float eps) {
+    const float* __restrict__ S0, const float* __restrict__ N0, const float* __restrict__ start_m,
+    const float* __restrict__ bias_i, const float* __restrict__ bias_f, const float* __restrict__ gain,
+    const int* __restrict__ item_len, const int* __restrict__ item_tok_off, const int* __restrict__ item_slot, int num_items,
+    MemoryShape sh, float cap, float q_scale, float eps) {
     extern __shared__ __attribute__((aligned(16))) float mem_lds[];
+    using L = MemoryOutLds<KQ, NV>;
     const int head = blockIdx.x, idx = blockIdx.y, tid = threadIdx.x;
     int item, chunk;
     if (!memory_find_chunk(idx, item_len, item_slot, num_items, item, chunk)) return;
@@ -352,50 +411,58 @@ __global__ __launch_bounds__(256) void memory_out_kernel(
     const int64_t row0 = (int64_t)item_tok_off[item] + (int64_t)chunk * kMemChunk;
     const float* p = proj + row0 * stride;
     const int dk = sh.dk, dv = sh.dv;
-    constexpr int KW = 4 * KQ, KS = KW + 4, VS = 68;
     double* sc = reinterpret_cast<double*>(mem_lds);           // c_j
     double* sM = sc + kMemChunk;                               // M_j
     float* sm = reinterpret_cast<float*>(sM + kMemChunk);      // m_j = F_j + M_j
     float* ks = sm + kMemChunk;
-    float* vs = ks + kMemChunk * KS;
+    float* vs = ks + L::first;
     const int64_t at = (int64_t)idx * sh.heads + head;
-    const float m0 = start_m[at];
-    if (tid < 64) {
-        double F, c, last;
-        memory_chunk_gates(F, c, last, p, stride, bias_i, bias_f, sh, head, n, cap);
-        double M = c;
-#pragma unroll
-        for (int o = 1; o < 64; o <<= 1) {
-            const double up = __shfl_up(M, o, 64);
-            if (tid >= o) M = fmax(M, up);
-        }
-        M = fmax(M, (double)m0);
-        sc[tid] = c;
-        sM[tid] = M;
-        sm[tid] = (float)(F + M);
-        // the request's last row leaves its maximum in the slot (the carry has read the old one)
-        if (tid == n - 1 && (chunk + 1) * kMemChunk >= item_len[item])
-            state[(int64_t)item_slot[item] * slot_stride + sh.m_base() + head] = (float)(F + M);
-    }
-    for (int e = tid; e < kMemChunk * KW; e += 256) {
-        const int j = e / KW, kk = e - j * KW;
-        ks[j * KS + kk] = (j < n && kk < dk) ? p[(int64_t)j * stride + sh.k_off() + (int64_t)head * dk + kk] : 0.f;
-    }
     const int lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
     const int i = wave * 16 + r16;                             // this lane's row of the chunk
     const bool row_ok = i < n;
-    float qf[KQ];
+    const float m0 = start_m[at];
     {
-        const float* qr = p + (int64_t)(row_ok ? i : 0) * stride + (int64_t)head * dk + g * KQ;
+        Tile<KQ> tk;
+        Tile<4 * NV> tv;
+        tk.template load<VEC>(p + sh.k_off() + (int64_t)head * dk, stride, n, 0, dk);
+        tv.template load<VEC>(p + sh.v_off() + (int64_t)head * dv, stride, n, 0, dv);
+        if (tid < 64) {
+            double F, c, last;
+            memory_chunk_gates(F, c, last, p, stride, bias_i, bias_f, sh, head, n, cap);
+            double M = c;
 #pragma unroll
-        for (int s = 0; s < KQ; ++s) qf[s] = (row_ok && g * KQ + s < dk) ? qr[s] * q_scale : 0.f;
+            for (int o = 1; o < 64; o <<= 1) {
+                const double up = __shfl_up(M, o, 64);
+                if (tid >= o) M = fmax(M, up);
+            }
+            M = fmax(M, (double)m0);
+            sc[tid] = c;
+            sM[tid] = M;
+            sm[tid] = (float)(F + M);
+            // the request's last row leaves its maximum in the slot (the carry has read the old one)
+            if (tid == n - 1 && (chunk + 1) * kMemChunk >= item_len[item])
+                state[(int64_t)item_slot[item] * slot_stride + sh.m_base() + head] = (float)(F + M);
+        }
+        tk.store(ks, L::KS);
+        tv.store(vs, L::VS);
     }
+    float qf[KQ];
     float den = 0.f;                                           // q . n_0, this lane group's share
     {
-        const float* n0 = N0 + at * dk + g * KQ;
+        const float* qr = p + (int64_t)min(i, n - 1) * stride + (int64_t)head * dk;
+        const float* n0 = N0 + at * dk;
 #pragma unroll
-        for (int s = 0; s < KQ; ++s) den = fmaf(qf[s], g * KQ + s < dk ? n0[s] : 0.f, den);
+        for (int s = 0; s < KQ; ++s) {
+            const int kk = 4 * s + g;
+            const float x = qr[min(kk, dk - 1)], y = n0[min(kk, dk - 1)];
+            qf[s] = row_ok && kk < dk ? x * q_scale : 0.f;
+            den = fmaf(qf[s], kk < dk ? y : 0.f, den);
+        }
     }
+    // the start state's first 64 key channels, on their way during the scores
+    const float* s0 = S0 + at * dk * dv;
+    Tile<4 * NV> ts;
+    ts.template load<VEC>(s0, dv, min(dk, 64), 0, dv);
     __syncthreads();
     const double Mi = sM[i];
     const float carried = expf((float)((double)m0 - Mi));
@@ -403,18 +470,12 @@ __global__ __launch_bounds__(256) void memory_out_kernel(
     // scores against the keys of this row's past in the chunk, weighted
     floatx4 st[4];
 #pragma unroll
-    for (int t = 0; t < 4; ++t) st[t] = floatx4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
     for (int t = 0; t < 4; ++t) {
+        st[t] = floatx4{0.f, 0.f, 0.f, 0.f};
         if (t > wave || 16 * t >= n) continue;                 // uniform over the wave
 #pragma unroll
-        for (int s = 0; s < KQ; s += 4) {
-            const float4 k4 = *reinterpret_cast<const float4*>(ks + (16 * t + r16) * KS + g * KQ + s);
-            st[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.x, qf[s], st[t], 0, 0, 0);
-            st[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.y, qf[s + 1], st[t], 0, 0, 0);
-            st[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.z, qf[s + 2], st[t], 0, 0, 0);
-            st[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.w, qf[s + 3], st[t], 0, 0, 0);
-        }
+        for (int s = 0; s < KQ; ++s)
+            st[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(ks[(16 * t + r16) * L::KS + 4 * s + g], qf[s], st[t], 0, 0, 0);
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int j = 16 * t + 4 * g + r;
@@ -428,40 +489,32 @@ __global__ __launch_bounds__(256) void memory_out_kernel(
 #pragma unroll
     for (int vt = 0; vt < NV; ++vt) o[vt] = floatx4{0.f, 0.f, 0.f, 0.f};
     // what the chunk's start state gives: o = S_0^T q, then times the row's factor
-    const float* s0 = S0 + at * dk * dv;
 #pragma unroll
-    for (int s = 0; s < KQ; ++s) {
-        const int kk = g * KQ + s;
-        const float* sr = s0 + (int64_t)min(kk, dk - 1) * dv;
+    for (int b = 0; b < (KQ + 15) / 16; ++b) {
+        if (64 * b >= dk) continue;
+        __syncthreads();                                       // the keys (or the channels before) have been read
+        ts.store(ks, L::SS);
+        __syncthreads();
+        if (64 * (b + 1) < dk) ts.template load<VEC>(s0 + (int64_t)64 * (b + 1) * dv, dv, min(dk - 64 * (b + 1), 64), 0, dv);
 #pragma unroll
-        for (int vt = 0; vt < NV; ++vt) {
-            const int col = 16 * vt + r16;
-            const float x = sr[min(col, dv - 1)];
-            o[vt] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk < dk && col < dv ? x : 0.f, qf[s], o[vt], 0, 0, 0);
+        for (int s = 0; s < (KQ < 16 ? KQ : 16); ++s) {
+            const float* sr = ks + (4 * s + g) * L::SS + r16;
+#pragma unroll
+            for (int vt = 0; vt < NV; ++vt)
+                o[vt] = __builtin_amdgcn_mfma_f32_16x16x4f32(sr[16 * vt], qf[(16 * b + s) % KQ], o[vt], 0, 0, 0);
         }
     }
 #pragma unroll
     for (int vt = 0; vt < NV; ++vt) o[vt] *= carried;
 #pragma unroll
-    for (int b = 0; b < (NV + 3) / 4; ++b) {                   // blocks of 64 value channels through LDS
-        if (64 * b >= dv) continue;
-        if (b) __syncthreads();                                // the block before has been read
-        for (int e = tid; e < kMemChunk * 64; e += 256) {
-            const int j = e >> 6, col = 64 * b + (e & 63);
-            vs[j * VS + (e & 63)] = (j < n && col < dv) ? p[(int64_t)j * stride + sh.v_off() + (int64_t)head * dv + col] : 0.f;
-        }
-        __syncthreads();
+    for (int t = 0; t < 4; ++t) {
+        if (t > wave || 16 * t >= n) continue;
 #pragma unroll
-        for (int t = 0; t < 4; ++t) {
-            if (t > wave || 16 * t >= n) continue;
+        for (int r = 0; r < 4; ++r) {
+            const float* vr = vs + (16 * t + 4 * g + r) * L::VS + r16;
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const float* vr = vs + (16 * t + 4 * g + r) * VS + r16;
-#pragma unroll
-                for (int vt = 0; vt < 4; ++vt)
-                    if (4 * b + vt < NV)
-                        o[(4 * b + vt) % NV] = __builtin_amdgcn_mfma_f32_16x16x4f32(vr[16 * vt], st[t][r], o[(4 * b + vt) % NV], 0, 0, 0);
-            }
+            for (int vt = 0; vt < NV; ++vt)
+                o[vt] = __builtin_amdgcn_mfma_f32_16x16x4f32(vr[16 * vt], st[t][r], o[vt], 0, 0, 0);
         }
     }
     // o[vt][r]: value channel 16 vt + 4 g + r of row i
@@ -484,12 +537,9 @@ __global__ __launch_bounds__(256) void memory_out_kernel(
     for (int vt = 0; vt < NV; ++vt) {
         const int v0 = 16 * vt + 4 * g;
         if (v0 >= dv) continue;
-        float y[4];
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int v = min(v0 + r, dv - 1);
-            y[r] = o[vt][r] * rms * gn[v] / (1.f + expf(-gate[v]));
-        }
+        const float4 z = load_piece<VEC>(gate, v0, dv, true), w = load_piece<VEC>(gn, v0, dv, true);
+        const float y[4] = {o[vt][0] * rms * w.x / (1.f + expf(-z.x)), o[vt][1] * rms * w.y / (1.f + expf(-z.y)),
+                            o[vt][2] * rms * w.z / (1.f + expf(-z.z)), o[vt][3] * rms * w.w / (1.f + expf(-z.w))};
         if (whole) Elem<T>::store4(dst + v0, y);
         else
             for (int r = 0; r < 4 && v0 + r < dv; ++r) Elem<T>::store(dst + v0 + r, y[r]);
@@ -509,6 +559,19 @@ static int memory_check(const MemoryShape& sh, int64_t stride, int64_t slot_stri
     ST_CHECK(slot_stride >= sh.slot(), "matrix_memory: a slot of %lld floats is smaller than the state (%lld)",
              (long long)slot_stride, (long long)sh.slot());
     ST_CHECK(cap > 0.f && eps > 0.f, "matrix_memory: the gates' cap and eps must be positive");
+    return 0;
+}
+
+// Kernels with more LDS than a launch may ask for by default have their limit raised, once each.
+static int raise_lds(const void* kernel, size_t bytes) {
+    static std::mutex mutex;
+    static std::set<const void*> raised;
+    if (bytes <= 48 * 1024) return 0;
+    std::lock_guard<std::mutex> lock(mutex);
+    if (raised.count(kernel)) return 0;
+    ST_CHECK(hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes) == hipSuccess,
+             "memory_chunks: cannot raise the LDS limit to %zu bytes", bytes);
+    raised.insert(kernel);
     return 0;
 }
 
@@ -564,35 +627,41 @@ extern "C" int st_memory_chunks(void* out, const float* proj, int64_t stride, fl
     ST_CHECK(scratch_chunks >= chunks, "memory_chunks: scratch for %lld chunks, %lld needed", (long long)scratch_chunks,
              (long long)chunks);
     ST_CHECK(chunks <= 65535 && num_items <= 65535, "memory_chunks: too many chunks or items");
-    const int kw = (key_dim + 15) / 16 * 16;
-    const size_t lds1 = sizeof(float) * ((size_t)kMemChunk * (kw + 4) + kMemChunk * 68 + kMemChunk);
-    static bool raised1 = false;
-    if (lds1 > 48 * 1024 && !raised1) {
-        ST_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(memory_sums_kernel), hipFuncAttributeMaxDynamicSharedMemorySize,
-                                     96 * 1024) == hipSuccess, "memory_chunks: cannot raise the LDS limit");
-        raised1 = true;
-    }
-    memory_sums_kernel<<<dim3(heads, (unsigned)chunks, (value_dim + 63) / 64), 256, lds1, stream>>>(
-        scratch_u, scratch_n, scratch_s, proj, stride, bias_i, bias_f, item_len, item_tok_off, item_slot, num_items, sh, cap);
+    // 16-byte loads where every section of a row and every row of the state starts on a 16-byte border
+    const bool vec = key_dim % 4 == 0 && value_dim % 4 == 0 && stride % 4 == 0 &&
+                     (((uintptr_t)proj | (uintptr_t)scratch_u | (uintptr_t)gain) & 15) == 0;
+    const dim3 grid1(heads, (unsigned)chunks, (value_dim + 63) / 64);
+#define ST_MS2(KQ, VEC)                                                                                                \
+    do {                                                                                                               \
+        auto kernel = memory_sums_kernel<KQ, VEC>;                                                                      \
+        const size_t lds = sizeof(float) * (size_t)(kMemChunk * (4 * KQ + 4) + kMemChunk * 68 + kMemChunk);              \
+        if (raise_lds(reinterpret_cast<const void*>(kernel), lds)) return 1;                                            \
+        kernel<<<grid1, 256, lds, stream>>>(scratch_u, scratch_n, scratch_s, proj, stride, bias_i, bias_f, item_len,     \
+                                            item_tok_off, item_slot, num_items, sh, cap);                               \
+    } while (0)
+#define ST_MS1(KQ) do { if (vec) ST_MS2(KQ, true); else ST_MS2(KQ, false); } while (0)
+    if (key_dim <= 16) ST_MS1(4);
+    else if (key_dim <= 32) ST_MS1(8);
+    else if (key_dim <= 64) ST_MS1(16);
+    else if (key_dim <= 128) ST_MS1(32);
+    else ST_MS1(64);
+#undef ST_MS1
+#undef ST_MS2
     ST_LAUNCH_CHECK("memory_chunks (sums)");
     const int elements = key_dim * value_dim + key_dim;
     memory_carry_kernel<<<dim3(heads, num_items, (elements + 255) / 256), 256, 0, stream>>>(
         scratch_u, scratch_n, scratch_s, scratch_m, state, slot_stride, item_len, item_slot, sh);
     ST_LAUNCH_CHECK("memory_chunks (carry)");
     const dim3 grid(heads, (unsigned)chunks);
-#define ST_MO(T, KQ, NV)                                                                                               \
+#define ST_MO_E(T, KQ, NV, VEC)                                                                                        \
     do {                                                                                                               \
-        auto kernel = memory_out_kernel<T, KQ, NV>;                                                                     \
-        const size_t lds = sizeof(double) * 2 * kMemChunk + sizeof(float) * (size_t)(kMemChunk + kMemChunk * (4 * KQ + 4) + kMemChunk * 68); \
-        static bool raised = false;                                                                                     \
-        if (lds > 48 * 1024 && !raised) {                                                                               \
-            ST_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, \
-                                         96 * 1024) == hipSuccess, "memory_chunks: cannot raise the LDS limit");         \
-            raised = true;                                                                                              \
-        }                                                                                                               \
+        auto kernel = memory_out_kernel<T, KQ, NV, VEC>;                                                                \
+        constexpr size_t lds = MemoryOutLds<KQ, NV>::bytes;                                                             \
+        if (raise_lds(reinterpret_cast<const void*>(kernel), lds)) return 1;                                            \
         kernel<<<grid, 256, lds, stream>>>((T*)out, proj, stride, state, slot_stride, scratch_u, scratch_n, scratch_m, bias_i, \
-            bias_f, gain, item_len, item_tok_off, item_slot, num_items, sh, cap, q_scale, eps);                                       \
+            bias_f, gain, item_len, item_tok_off, item_slot, num_items, sh, cap, q_scale, eps);                         \
     } while (0)
+#define ST_MO(T, KQ, NV) do { if (vec) ST_MO_E(T, KQ, NV, true); else ST_MO_E(T, KQ, NV, false); } while (0)
 #define ST_MO_V(T, KQ) do { if (value_dim <= 64) ST_MO(T, KQ, 4); else if (value_dim <= 128) ST_MO(T, KQ, 8); else ST_MO(T, KQ, 16); } while (0)
 #define ST_MO_K(T) do { if (key_dim <= 16) ST_MO_V(T, 4); else if (key_dim <= 32) ST_MO_V(T, 8); else if (key_dim <= 64) ST_MO_V(T, 16); \
                         else if (key_dim <= 128) ST_MO_V(T, 32); else ST_MO_V(T, 64); } while (0)
@@ -600,6 +669,7 @@ extern "C" int st_memory_chunks(void* out, const float* proj, int64_t stride, fl
 #undef ST_MO_K
 #undef ST_MO_V
 #undef ST_MO
+#undef ST_MO_E
     ST_LAUNCH_CHECK("memory_chunks (outputs)");
     return 0;
 }

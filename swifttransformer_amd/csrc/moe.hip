@@ -11,18 +11,21 @@
 //   down     per tile and 64 output features: the output product; with one expert a token the
 //            result goes straight into the residual stream, otherwise to a row per pair that
 //   combine  sums in the order of the token's choices.
-// A wave computes a 16 x 16 block of results with operands read straight from memory in the
+// A wave computes 16 x 16 blocks of results with operands read straight from memory in the
 // matrix instruction's own layout (16 bytes a lane and step): with 16 rows a tile the products
 // are bound by the stream of expert weights, which every tile reads once.
 #include "api.h"
 #include "common.h"
 #include "activation.h"
 
+#include <type_traits>
+
 namespace st {
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float floatx4 __attribute__((ext_vector_type(4)));
 
+template <int N> using Steps = std::integral_constant<int, N>;
 constexpr int kRows = 16;            // rows of one matrix-instruction block
 constexpr int kMaxTop = 16;
 
@@ -189,6 +192,7 @@ template <typename T> struct Frag;
 template <> struct Frag<bf16_t> {
     static constexpr int kDepth = 32, kLane = 8;
     bf16x8 v;
+    __device__ inline void load_whole(const bf16_t* p) { v = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(p)); }
     __device__ inline void load(const bf16_t* row, int k, int K, bool ok, bool vec) {
         if (ok && vec && k + 8 <= K) {
             v = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(row + k));
@@ -207,6 +211,10 @@ template <> struct Frag<bf16_t> {
 template <> struct Frag<float> {
     static constexpr int kDepth = 16, kLane = 4;
     float v[4];
+    __device__ inline void load_whole(const float* p) {
+        const float4 x = *reinterpret_cast<const float4*>(p);
+        v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w;
+    }
     __device__ inline void load(const float* row, int k, int K, bool ok, bool vec) {
         if (ok && vec && k + 4 <= K) {
             const float4 x = *reinterpret_cast<const float4*>(row + k);
@@ -223,10 +231,136 @@ template <> struct Frag<float> {
     }
 };
 
+// ---- few rows an expert: tiles of 16 places, where only the weights' stream counts.  A workgroup takes 16 features; its
+// four waves share the depth, so that a wave's part is one or a few batches of loads that are all on their way at once and
+// that the waves' rows, which lie a whole row of weights apart, start at different offsets (equal offsets meet in the
+// same memory channels); the waves' sums meet in LDS.  The addresses of rows and features that do not exist stand for
+// row and feature 0: their results are not stored.
+template <typename T, int MATS>
+__device__ inline void moe_depth_share(floatx4* acc, const T* xr, const T* const* wr, int K, int vec) {
+    constexpr int D = Frag<T>::kDepth, L = Frag<T>::kLane;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4;
+    const int steps = (K + D - 1) / D, share = (steps + 3) / 4;
+    int k0 = wave * share * D;
+    const int end = min(K, k0 + share * D);
+    auto batches = [&](auto count) {
+        constexpr int U = decltype(count)::value;
+        for (; k0 + U * D <= end; k0 += U * D) {
+            Frag<T> a[U], b[MATS][U];
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int k = k0 + u * D + L * g;
+#pragma unroll
+                for (int m = 0; m < MATS; ++m) b[m][u].load_whole(wr[m] + k);
+                a[u].load_whole(xr + k);
+            }
+            __builtin_amdgcn_sched_barrier(0);    // (left to itself the compiler keeps a few of the loads on their way)
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+#pragma unroll
+                for (int m = 0; m < MATS; ++m) acc[m] = Frag<T>::mma(a[u], b[m][u], acc[m]);
+        }
+    };
+    if (vec) {
+        batches(Steps<MATS == 1 ? 16 : 8>());
+        batches(Steps<4>());
+    }
+    for (; k0 < end; k0 += D) {
+        Frag<T> a, b;
+        a.load(xr, k0 + L * g, K, true, vec);
+#pragma unroll
+        for (int m = 0; m < MATS; ++m) {
+            b.load(wr[m], k0 + L * g, K, true, vec);
+            acc[m] = Frag<T>::mma(a, b, acc[m]);
+        }
+    }
+}
+
+// the waves' blocks of 16 x 16 summed: thread t of the workgroup gets row t / 16, feature t % 16
+template <int MATS>
+__device__ inline void moe_sum_shares(float* sum, const floatx4* acc, float* lds) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+#pragma unroll
+    for (int m = 0; m < MATS; ++m) *reinterpret_cast<floatx4*>(lds + ((wave * MATS + m) * 64 + lane) * 4) = acc[m];
+    __syncthreads();
+    const int row = threadIdx.x >> 4, from = ((row >> 2) * 16 + (threadIdx.x & 15)) * 4 + (row & 3);
+#pragma unroll
+    for (int m = 0; m < MATS; ++m) {
+        sum[m] = 0.f;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) sum[m] += lds[(w * MATS + m) * 256 + from];
+    }
+}
+
+// grid (tiles, ceil(inner / 16))
+template <typename T, bool GATED>
+__global__ __launch_bounds__(256) void moe_up_few_kernel(
+    T* __restrict__ y, const T* __restrict__ x, const T* __restrict__ w_gate, const T* __restrict__ w_up,
+    const int* __restrict__ sorted, const int* __restrict__ tile_expert, const float* __restrict__ weights,
+    int top, int width, int inner, float limit, int style, int vec) {
+    constexpr int MATS = GATED ? 2 : 1;
+    __shared__ __attribute__((aligned(16))) float lds[4 * MATS * 256];
+    const int tile = blockIdx.x, e = tile_expert[tile];
+    if (e < 0) return;
+    const int r16 = threadIdx.x & 15, f0 = blockIdx.y * 16, base = tile * kRows;
+    const int64_t feature = (int64_t)e * inner + min(f0 + r16, inner - 1);
+    const int pair = sorted[base + r16];
+    const T* wr[MATS];
+    wr[0] = w_up + feature * width;
+    if (GATED) wr[MATS - 1] = w_gate + feature * width;
+    floatx4 acc[MATS];
+#pragma unroll
+    for (int m = 0; m < MATS; ++m) acc[m] = floatx4{0.f, 0.f, 0.f, 0.f};
+    moe_depth_share<T, MATS>(acc, x + (int64_t)(pair >= 0 ? pair / top : 0) * width, wr, width, vec);
+    float sum[MATS];
+    moe_sum_shares<MATS>(sum, acc, lds);
+    const int place = base + (threadIdx.x >> 4), f = f0 + r16;
+    if (f >= inner) return;
+    const int p = sorted[place];
+    float out = 0.f;
+    if (p >= 0 && !GATED) {
+        out = apply_activation(kActGeluErf, sum[0]);
+    } else if (p >= 0 && style == 1) {
+        const float gv = sum[MATS - 1];
+        out = gv / (1.f + expf(-gv)) * sum[0];
+    } else if (p >= 0) {
+        const float s = weights[p];
+        const float gv = fminf(s * sum[MATS - 1], limit);
+        const float uv = fminf(fmaxf(s * sum[0], -limit), limit);
+        out = gv / (1.f + expf(-1.702f * gv)) * (uv + 1.f);
+    }
+    Elem<T>::store(y + (int64_t)place * inner + f, out);
+}
+
+// grid (tiles, ceil(width / 16))
+template <typename T>
+__global__ __launch_bounds__(256) void moe_down_few_kernel(
+    float* out, const float* residual, float* __restrict__ pair_out, const T* __restrict__ y, const T* __restrict__ w_down,
+    const int* __restrict__ sorted, const int* __restrict__ tile_expert, int top, int width, int inner, float out_scale,
+    int vec) {
+    __shared__ __attribute__((aligned(16))) float lds[4 * 256];
+    const int tile = blockIdx.x, e = tile_expert[tile];
+    if (e < 0) return;
+    const int r16 = threadIdx.x & 15, n0 = blockIdx.y * 16, base = tile * kRows;
+    const T* wr[1] = {w_down + ((int64_t)e * width + min(n0 + r16, width - 1)) * inner};
+    floatx4 acc[1] = {floatx4{0.f, 0.f, 0.f, 0.f}};
+    moe_depth_share<T, 1>(acc, y + (int64_t)(base + r16) * inner, wr, inner, vec);
+    float sum[1];
+    moe_sum_shares<1>(sum, acc, lds);
+    const int place = base + (threadIdx.x >> 4), n = n0 + r16;
+    const int p = sorted[place];
+    if (n >= width || p < 0) return;
+    if (pair_out) {
+        pair_out[(int64_t)place * width + n] = sum[0];
+    } else {                                           // one expert a token: p is the token
+        const int64_t at = (int64_t)p * width + n;
+        out[at] = fmaf(out_scale, sum[0], residual[at]);
+    }
+}
+
 // grid (tiles, ceil(inner / 64)); wave w of the workgroup takes inner features f0 + 16 w .. +15 of
 // the tile's RT blocks of 16 rows: a step's weight operands are loaded once and meet RT blocks of
-// rows (RT = 1 for few rows an expert, where only the weights' stream counts; RT = 4 or 8 for
-// prompts, where every tile reads its expert's weights again from the L2).
+// rows (4 or 8, for prompts, where every tile reads its expert's weights again from the L2).
 // Result layout of a block: lane (r16, g) holds rows 4g .. 4g+3 of feature r16.
 // GATED false: one weight matrix (w_up) and the exact GELU of its product (style 2).
 template <typename T, int RT, bool GATED>
@@ -256,7 +390,32 @@ __global__ __launch_bounds__(256) void moe_up_kernel(
     for (int b = 0; b < RT; ++b) { cg[b] = floatx4{0.f, 0.f, 0.f, 0.f}; cu[b] = floatx4{0.f, 0.f, 0.f, 0.f}; }
     constexpr int D = Frag<T>::kDepth, L = Frag<T>::kLane;
 
-    for (int k0 = 0; k0 < width; k0 += D) {
+    // (the addresses of rows and features that do not exist stand for row and feature 0: their results are not stored)
+    int k0 = 0;
+    auto batches = [&](auto steps) {
+        constexpr int U = decltype(steps)::value;
+        for (; k0 + U * D <= width; k0 += U * D) {
+            Frag<T> a[U][RT], bg[U], bu[U];
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int k = k0 + u * D + L * g;
+                if (GATED) bg[u].load_whole(gr + k);
+                bu[u].load_whole(ur + k);
+#pragma unroll
+                for (int b = 0; b < RT; ++b) a[u][b].load_whole(xr[b] + k);
+            }
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+#pragma unroll
+                for (int b = 0; b < RT; ++b) {
+                    if (GATED) cg[b] = Frag<T>::mma(a[u][b], bg[u], cg[b]);
+                    cu[b] = Frag<T>::mma(a[u][b], bu[u], cu[b]);
+                }
+        }
+    };
+    if (vec && RT == 4) batches(Steps<2>());
+    for (; k0 < width; k0 += D) {
         Frag<T> a[RT], bg, bu;
         const int k = k0 + L * g;
         if (GATED) bg.load(gr, k, width, f_ok, vec);
@@ -312,7 +471,27 @@ __global__ __launch_bounds__(256) void moe_down_kernel(
     for (int b = 0; b < RT; ++b) c[b] = floatx4{0.f, 0.f, 0.f, 0.f};
     constexpr int D = Frag<T>::kDepth, L = Frag<T>::kLane;
 
-    for (int k0 = 0; k0 < inner; k0 += D) {
+    int k0 = 0;
+    auto batches = [&](auto steps) {              // (as in moe_up_kernel)
+        constexpr int U = decltype(steps)::value;
+        for (; k0 + U * D <= inner; k0 += U * D) {
+            Frag<T> a[U][RT], bw[U];
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int k = k0 + u * D + L * g;
+                bw[u].load_whole(wr + k);
+#pragma unroll
+                for (int b = 0; b < RT; ++b) a[u][b].load_whole(yr + (int64_t)b * kRows * inner + k);
+            }
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+#pragma unroll
+                for (int b = 0; b < RT; ++b) c[b] = Frag<T>::mma(a[u][b], bw[u], c[b]);
+        }
+    };
+    if (vec && RT == 4) batches(Steps<2>());
+    for (; k0 < inner; k0 += D) {
         Frag<T> a[RT], bw;
         const int k = k0 + L * g;
         bw.load(wr, k, inner, n_ok, vec);
@@ -496,25 +675,49 @@ __global__ __launch_bounds__(256) void moe_tiled_kernel(
     }
 }
 
+// V columns a thread and turn (4: 16-byte accesses)
+template <int V>
 __global__ __launch_bounds__(256) void moe_combine_kernel(
-    float* __restrict__ out, const float* __restrict__ residual, const float* __restrict__ pair_out,
+    float* out, const float* residual, const float* __restrict__ pair_out,
     const int* __restrict__ place_of_pair, const float* __restrict__ weights, int top, int width, float out_scale) {
     const int t = blockIdx.x;
-    for (int n = threadIdx.x; n < width; n += 256) {
-        float sum = 0.f;
+    for (int n = threadIdx.x * V; n < width; n += 256 * V) {
+        float sum[V], base[V];
         bool any = false;
+        const int64_t at = (int64_t)t * width + n;
+#pragma unroll
+        for (int v = 0; v < V; ++v) { sum[v] = 0.f; base[v] = 0.f; }
+        if (residual) {
+            if (V == 4) {
+                const float4 r = *reinterpret_cast<const float4*>(residual + at);
+                base[0] = r.x; base[1 % V] = r.y; base[2 % V] = r.z; base[3 % V] = r.w;
+            } else {
+                base[0] = residual[at];
+            }
+        }
+#pragma unroll 2
         for (int j = 0; j < top; ++j) {
             const int place = place_of_pair[(int64_t)t * top + j];
+            const float w = weights ? weights[(int64_t)t * top + j] : 1.f;
+            const float* src = pair_out + (int64_t)max(place, 0) * width + n;
+            float x[V];
+            if (V == 4) {
+                const float4 r = *reinterpret_cast<const float4*>(src);
+                x[0] = r.x; x[1 % V] = r.y; x[2 % V] = r.z; x[3 % V] = r.w;
+            } else {
+                x[0] = src[0];
+            }
             if (place >= 0) {
-                const float v = pair_out[(int64_t)place * width + n];
-                sum = weights ? fmaf(weights[(int64_t)t * top + j], v, sum) : sum + v;
+#pragma unroll
+                for (int v = 0; v < V; ++v) sum[v] = fmaf(w, x[v], sum[v]);
                 any = true;
             }
         }
-        const int64_t at = (int64_t)t * width + n;
-        if (!residual) out[at] = any ? out_scale * sum : 0.f;
-        else if (any) out[at] = fmaf(out_scale, sum, residual[at]);
-        else if (out != residual) out[at] = residual[at];
+        if (residual && !any && out == residual) continue;
+#pragma unroll
+        for (int v = 0; v < V; ++v) sum[v] = any ? fmaf(out_scale, sum[v], base[v]) : base[v];
+        if (V == 4) *reinterpret_cast<float4*>(out + at) = make_float4(sum[0], sum[1 % V], sum[2 % V], sum[3 % V]);
+        else out[at] = sum[0];
     }
 }
 
@@ -596,9 +799,22 @@ extern "C" int st_moe_up(void* y, const void* x, const void* w_gate, const void*
 #define ST_UP_G(T, RT, G)                                                                                    \
     moe_up_kernel<T, RT, G><<<grid, 256, 0, stream>>>((T*)y, (const T*)x, (const T*)w_gate, (const T*)w_up, sorted, \
                                                       tile_expert, weights, top, width, inner, limit, style, vec)
+    if (tile == 16) {
+        const dim3 few(capacity / 16, (inner + 15) / 16);
+        ST_CHECK(few.y <= 65535, "moe_up: too many inner features");
+#define ST_UP_FEW(T, G)                                                                                      \
+    moe_up_few_kernel<T, G><<<few, 256, 0, stream>>>((T*)y, (const T*)x, (const T*)w_gate, (const T*)w_up, sorted, tile_expert, \
+                                                     weights, top, width, inner, limit, style, vec)
+        if (dtype == kF32) { if (style == 2) ST_UP_FEW(float, false); else ST_UP_FEW(float, true); }
+        else if (dtype == kBF16) { if (style == 2) ST_UP_FEW(bf16_t, false); else ST_UP_FEW(bf16_t, true); }
+        else ST_CHECK(false, "moe_up: unknown dtype %d", dtype);
+#undef ST_UP_FEW
+        ST_LAUNCH_CHECK("moe_up (few rows)");
+        return 0;
+    }
 #define ST_UP(T, RT) do { if (style == 2) ST_UP_G(T, RT, false); else ST_UP_G(T, RT, true); } while (0)
-    if (dtype == kF32) { if (tile == 16) ST_UP(float, 1); else if (tile == 64) ST_UP(float, 4); else ST_UP(float, 8); }
-    else if (dtype == kBF16) { if (tile == 16) ST_UP(bf16_t, 1); else if (tile == 64) ST_UP(bf16_t, 4); else ST_UP(bf16_t, 8); }
+    if (dtype == kF32) { if (tile == 64) ST_UP(float, 4); else ST_UP(float, 8); }
+    else if (dtype == kBF16) { if (tile == 64) ST_UP(bf16_t, 4); else ST_UP(bf16_t, 8); }
     else ST_CHECK(false, "moe_up: unknown dtype %d", dtype);
 #undef ST_UP
 #undef ST_UP_G
@@ -625,11 +841,24 @@ extern "C" int st_moe_down(float* out, const float* residual, float* pair_out, c
         ST_LAUNCH_CHECK("moe_down (tiled)");
         return 0;
     }
+    if (tile == 16) {
+        const dim3 few(capacity / 16, (width + 15) / 16);
+        ST_CHECK(few.y <= 65535, "moe_down: too wide");
+#define ST_DOWN_FEW(T)                                                                                       \
+    moe_down_few_kernel<T><<<few, 256, 0, stream>>>(out, residual, pair_out, (const T*)y, (const T*)w_down, sorted, tile_expert, \
+                                                    top, width, inner, out_scale, vec)
+        if (dtype == kF32) ST_DOWN_FEW(float);
+        else if (dtype == kBF16) ST_DOWN_FEW(bf16_t);
+        else ST_CHECK(false, "moe_down: unknown dtype %d", dtype);
+#undef ST_DOWN_FEW
+        ST_LAUNCH_CHECK("moe_down (few rows)");
+        return 0;
+    }
 #define ST_DOWN(T, RT)                                                                                        \
     moe_down_kernel<T, RT><<<grid, 256, 0, stream>>>(out, residual, pair_out, (const T*)y, (const T*)w_down,      \
                                                      sorted, tile_expert, top, width, inner, out_scale, vec)
-    if (dtype == kF32) { if (tile == 16) ST_DOWN(float, 1); else if (tile == 64) ST_DOWN(float, 4); else ST_DOWN(float, 8); }
-    else if (dtype == kBF16) { if (tile == 16) ST_DOWN(bf16_t, 1); else if (tile == 64) ST_DOWN(bf16_t, 4); else ST_DOWN(bf16_t, 8); }
+    if (dtype == kF32) { if (tile == 64) ST_DOWN(float, 4); else ST_DOWN(float, 8); }
+    else if (dtype == kBF16) { if (tile == 64) ST_DOWN(bf16_t, 4); else ST_DOWN(bf16_t, 8); }
     else ST_CHECK(false, "moe_down: unknown dtype %d", dtype);
 #undef ST_DOWN
     ST_LAUNCH_CHECK("moe_down");
@@ -642,7 +871,11 @@ extern "C" int st_moe_combine(float* out, const float* residual, const float* pa
     ST_CHECK(num_tokens >= 0 && top >= 1 && width > 0, "moe_combine: bad sizes");
     ST_CHECK(out && pair_out && place_of_pair, "moe_combine: null operand");
     if (num_tokens == 0) return 0;
-    moe_combine_kernel<<<num_tokens, 256, 0, stream>>>(out, residual, pair_out, place_of_pair, weights, top, width, out_scale);
+    const bool vec = width % 4 == 0 && (((uintptr_t)out | (uintptr_t)residual | (uintptr_t)pair_out) & 15) == 0;
+    if (vec)
+        moe_combine_kernel<4><<<num_tokens, 256, 0, stream>>>(out, residual, pair_out, place_of_pair, weights, top, width, out_scale);
+    else
+        moe_combine_kernel<1><<<num_tokens, 256, 0, stream>>>(out, residual, pair_out, place_of_pair, weights, top, width, out_scale);
     ST_LAUNCH_CHECK("moe_combine");
     return 0;
 }

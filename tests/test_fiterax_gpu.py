@@ -474,7 +474,7 @@ def test_a_memory_that_keeps_a_token_for_long(models, tmp_path, dtype):
     refs = {r: plain.logits(cfg, w, s).numpy() for r, s in seqs.items()}
     other = plain.logits(cfg, w, seqs[1][:60] + seqs[0][60:]).numpy()
     assert np.abs(other[299] - refs[0][299]).max() > 0.3 * refs[0][299].std()       # the first tokens show at the end
-    runner = make_runner(folder, dtype, 4, 4, record_after=2, max_seqs=2)
+    runner = make_runner(folder, dtype, 4, 120, record_after=2, max_seqs=2)
     run_schedule(runner, seqs, refs, [[(0, 40), (1, 2)]] + [[(0, 1), (1, 1)]] * 30 + [[(1, 70), (0, 1)], [(0, 2), (1, 18)], [(0, 150)]] +
                  [[(0, 1)]] * 77, dtype, "beside another", loosen=3.0)
 
