@@ -229,3 +229,44 @@ def fiterax_preset(name: str, **overrides):
                         embedding_scale=float(hidden) ** 0.5, residual_mult=0.5, max_positions=4096)
     fields.update(overrides)
     return FiteraxHyperParam(**fields).validate()
+
+
+# ---- named sizes of the Fefozen family, for runs with random weights: the layer sizes of the OPT model of the same
+# name.  Of every four layers the first two are gated delta rules (a quarter of the heads as query/key heads, keys and values
+# of the head size, four taps), the third a latent attention with a sink, the fourth one without (the second of these and so
+# on read the first one's cache in turn); latents of 128 for the cache and a quarter of the width for the queries, a turned
+# part of 32; dense feed-forwards of half the OPT inner width alternate with 14 experts of a quarter of it and 2 identity
+# experts, 2 a token.
+def fefozen_preset(name: str, **overrides):
+    from .fefozen_param import FefozenHyperParam
+    key = name.lower().replace("-", "_")
+    size = key.split("_", 1)[1] if "_" in key else ""
+    if "opt_" + size not in _SIZES:
+        raise KeyError(f"invalid model name {name!r}; valid names: " +
+                       " ".join("fefozen_" + k.split("_", 1)[1] for k in _SIZES))
+    n_layers, hidden, heads, ffn = _SIZES["opt_" + size]
+    n_layers = int(overrides.pop("num_layers", n_layers))
+    only = overrides.pop("only", None)            # one mixer type for every layer (measurements)
+    rank = int(overrides.pop("rank", 128))
+    hd = hidden // heads
+    layers, lender = [], None
+    for i in range(n_layers):
+        kind = only or ("delta", "delta", "latent_attention", "latent_attention_2")[i % 4]
+        if kind == "delta":
+            mixer = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": hd, "vdim": hd, "conv": 4}
+        else:
+            mixer = {"heads": heads, "dim": hd, "rot_dim": 32, "vdim": hd, "q_rank": hidden // 4, "kv_rank": rank,
+                     "scale": float(hd + 32) ** -0.5, "rot": {"dims": 32, "base": 500000.0}}
+            if kind == "latent_attention_2":
+                if lender is None:
+                    lender = i
+                else:
+                    mixer["kv_from"], lender = lender, None
+        if i % 2 == 0:
+            mlp = {"kind": "dense", "ff": ffn // 2}
+        else:
+            mlp = {"kind": "moe", "router": {"experts": 14, "identity": 2, "top": 2}, "expert": {"ff": ffn // 4, "limit": 7.0}}
+        layers.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    fields: Dict = dict(vocab=50272, width=hidden, layers=layers, norm_eps=1e-6, max_positions=4096)
+    fields.update(overrides)
+    return FefozenHyperParam(**fields).validate()

@@ -233,7 +233,7 @@ int st_latent_write(void* cache, int64_t page_stride, const float* x, int64_t x_
 // experts of the `keep` best of `groups` equal groups of neighbours (a group's rank: its largest logit) can be
 // chosen, mode 3 the sigmoid of each chosen logit over the chosen sigmoids' sum (+ 1e-20), times `scale`, where the
 // choice goes by sigmoid + correction [experts] (else null).  Rows whose item is -1 get ids of -1.
-int st_moe_route(int* ids, float* weights, const float* logits, const int* token_item, const float* correction,
+int st_moe_route(int* ids, float* weights, const float* logits, int logit_stride, const int* token_item, const float* correction,
                  float scale, int num_tokens, int experts, int top, int mode, int groups, int keep, hipStream_t stream);
 // Sorts the num_pairs = tokens * top (token, choice) pairs by expert into tiles of `tile` (16, 64 or 128)
 // places that hold one expert's pairs each: sorted[capacity] (pair index, or -1),
@@ -258,7 +258,8 @@ int st_moe_down(float* out, const float* residual, float* pair_out, const void* 
 // out[t, n] = residual[t, n] + out_scale * sum_j weights[t * top + j] * pair_out[place_of_pair[t * top + j], n]
 // (weights null: ones; residual null: zeros)
 int st_moe_combine(float* out, const float* residual, const float* pair_out, const int* place_of_pair,
-                   const float* weights, int num_tokens, int top, int width, float out_scale, hipStream_t stream);
+                   const float* weights, const int* ids, const void* x, int experts, int num_tokens, int top, int width,
+                   float out_scale, int dtype, hipStream_t stream);
 
 // ---- float operations on the residual stream (csrc/stream_ops.hip)
 // y = tanh(alpha[0] * x[row]) * w + b (b may be null) of every row, or of the rows picked by `rows`
@@ -331,6 +332,47 @@ int st_memory_chunks(void* out, const float* proj, int64_t stride, float* state,
                      const int* item_slot, int num_items, int num_rows, int heads, int key_dim, int value_dim, float cap,
                      float q_scale, float eps, float* scratch_u, float* scratch_n, double* scratch_s, float* scratch_m,
                      int64_t scratch_chunks, int dtype, hipStream_t stream);
+
+// ---- attention over a latent cache shared by all heads (csrc/latent_attention.hip, csrc/latent.hip)
+int st_latent_inputs(void* cq, int cq_width, const float* gain_q, int q_rank, void* cache, int64_t page_stride,
+                     const float* gain, int rank, int tail_off, int tail, const float* freq, int half, float tail_mult,
+                     int entry, const float* x, int64_t x_stride, const int* token_item, const int* positions,
+                     const int* block_table, int max_pages, int page_size, int num_tokens, float eps, int dtype,
+                     hipStream_t stream);
+int st_latent_max_entry();
+int st_latent_tiles(void* out, const void* q, int64_t q_stride, const void* cache, int64_t page_stride, const int* tile_item,
+                    const int* tile_q0, int num_tiles, const int* item_tok_off, const int* item_start, const int* item_len,
+                    const int* block_table, const float* sink, const float* freq, int max_pages, int page_size, int heads,
+                    int entry, int out_dim, int rot_off, int rot_half, float rot_mult, float scale, int window, int dtype,
+                    hipStream_t stream);
+int st_latent_rows(float* part_o, float* part_lse, const void* q, int64_t q_stride, const void* cache, int64_t page_stride,
+                   const int* row_ids, const int* token_item, const int* positions, int num_rows, int num_splits,
+                   const int* block_table, const float* sink, const float* freq, int max_pages, int page_size, int heads,
+                   int entry, int out_dim, int rot_off, int rot_half, float rot_mult, float scale, int window, int dtype,
+                   hipStream_t stream);
+int st_latent_merge(void* out, const float* part_o, const float* part_lse, const int* row_ids, int num_rows, int heads,
+                    int out_dim, int num_splits, int dtype, hipStream_t stream);
+int st_latent_up(void* y, const void* o, const float* part_o, const float* part_lse, int num_splits, const void* w,
+                 const float* gate, int64_t gate_stride, const int* token_item, int num_tokens, int heads, int value_dim,
+                 int out_dim, int dtype, hipStream_t stream);
+
+// ---- gated delta rule (csrc/delta.hip)
+int64_t st_delta_slot(int heads, int qk_heads, int key_dim, int value_dim, int taps);
+int st_delta_chunk_rows();
+int st_delta_step(void* out, const float* proj, int64_t stride, float* state, int64_t slot_stride, const float* taps_w,
+                  const float* a_log, const float* dt_bias, const float* gain, const int* positions, const int* item_len,
+                  const int* item_tok_off, const int* item_slot, int num_items, int heads, int qk_heads, int key_dim,
+                  int value_dim, int taps, float q_scale, float unit_eps, float eps, int dtype, hipStream_t stream);
+int st_delta_chunks(void* out, const float* proj, int64_t stride, float* state, int64_t slot_stride, const float* taps_w,
+                    const float* a_log, const float* dt_bias, const float* gain, const int* token_item, const int* positions,
+                    const int* item_len, const int* item_tok_off, const int* item_slot, int num_items, int num_rows, int heads,
+                    int qk_heads, int key_dim, int value_dim, int taps, float q_scale, float unit_eps, float eps, float* qkv,
+                    float* gates, float* wv, float* wk, float* kt, float* fall, float* start, int64_t scratch_chunks, int dtype,
+                    hipStream_t stream);
+
+// ---- a branch's result into the residual stream through a norm, and the next branch's input (csrc/residual_norm.hip)
+int st_rms_onto(float* out32, void* out_t, const float* y, const float* x, const float* gain, const float* gain2, int num_rows,
+                int width, float eps, float eps2, int dtype, hipStream_t stream);
 
 // Measurement kernels (csrc/probe.hip): a plain streaming read, and a kernel without work.
 int st_probe_read(const void* src, int64_t bytes, void* sink, int workgroups, int pattern, hipStream_t stream);

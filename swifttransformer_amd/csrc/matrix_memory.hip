@@ -22,6 +22,7 @@
 // A row of `proj` is q | k | v | g | zi | zf: (heads x dk) twice, (heads x dv) twice, heads twice, floats.
 // A slot is S [heads, dk, dv] | n [heads, dk] | m [heads].
 #include "api.h"
+#include "chunk_tiles.h"
 #include "common.h"
 
 #include <mutex>
@@ -31,7 +32,7 @@ namespace st {
 
 typedef float floatx4 __attribute__((ext_vector_type(4)));
 
-constexpr int kMemChunk = 64;
+constexpr int kMemChunk = kChunkRows;
 constexpr int kMemMaxDim = 256;
 
 __device__ inline float log_input_gate(float z, float cap) { return cap * tanhf(z / cap); }
@@ -161,23 +162,6 @@ __global__ __launch_bounds__(1024) void memory_step_kernel(
 }
 
 // ---------------------------------------------------------------- chunks
-// the chunk of an item that a global chunk index means; false past the last one
-__device__ inline bool memory_find_chunk(int idx, const int* __restrict__ item_len, const int* __restrict__ item_slot,
-                                         int num_items, int& item, int& chunk) {
-    int base = 0;
-    for (int b = 0; b < num_items; ++b) {
-        const int len = item_len[b];
-        const int n = (item_slot[b] >= 0 && len > 0) ? (len + kMemChunk - 1) / kMemChunk : 0;
-        if (idx < base + n) {
-            item = b;
-            chunk = idx - base;
-            return true;
-        }
-        base += n;
-    }
-    return false;
-}
-
 // The first wave: F_j (inclusive sums of the log forget gates) and c_j = i_j - F_j of a chunk's n rows; c = -inf past
 // them.  `last`: the chunk's whole sum F_(n-1).
 __device__ inline void memory_chunk_gates(double& F, double& c, double& last, const float* __restrict__ p, int64_t stride,
@@ -206,58 +190,6 @@ __device__ inline double wave_max_double(double v) {
     return v;
 }
 
-// Four neighbouring floats of a row, zeros past its `limit` numbers or where the row does not exist.  VEC: the row starts
-// on 16 bytes and the limit is a multiple of 4.  (Addresses are clamped and values cleared rather than loads behind a
-// branch: the loads of a tile are then all on their way at once.)
-template <bool VEC>
-__device__ inline float4 load_piece(const float* __restrict__ row, int c, int limit, bool ok) {
-    float4 v;
-    if (VEC) {
-        v = *reinterpret_cast<const float4*>(row + min(c, limit - 4));
-    } else {
-        v.x = row[min(c, limit - 1)];
-        v.y = row[min(c + 1, limit - 1)];
-        v.z = row[min(c + 2, limit - 1)];
-        v.w = row[min(c + 3, limit - 1)];
-    }
-    v.x = ok && c < limit ? v.x : 0.f;
-    v.y = ok && c + 1 < limit ? v.y : 0.f;
-    v.z = ok && c + 2 < limit ? v.z : 0.f;
-    v.w = ok && c + 3 < limit ? v.w : 0.f;
-    return v;
-}
-
-// A tile of 64 rows x 4 * P4 floats (P4 a power of two) by 256 threads: piece i of a thread is row e / P4, floats 4 (e % P4)
-// on, e = thread + 256 i; P4 / 4 pieces a thread.
-template <int P4>
-struct Tile {
-    static constexpr int kPieces = P4 / 4;
-    float4 v[kPieces];
-    template <bool VEC>
-    __device__ inline void load(const float* __restrict__ base, int64_t stride, int rows, int first, int limit) {
-#pragma unroll
-        for (int i = 0; i < kPieces; ++i) {
-            const int e = threadIdx.x + 256 * i, j = e / P4, c = 4 * (e % P4);
-            v[i] = load_piece<VEC>(base + (int64_t)min(j, rows - 1) * stride, first + c, limit, j < rows);
-        }
-    }
-    __device__ inline void store(float* lds, int lds_stride) const {
-#pragma unroll
-        for (int i = 0; i < kPieces; ++i) {
-            const int e = threadIdx.x + 256 * i;
-            *reinterpret_cast<float4*>(lds + (e / P4) * lds_stride + 4 * (e % P4)) = v[i];
-        }
-    }
-    __device__ inline void store_weighted(float* lds, int lds_stride, const float* w) const {
-#pragma unroll
-        for (int i = 0; i < kPieces; ++i) {
-            const int e = threadIdx.x + 256 * i;
-            const float f = w[e / P4];
-            *reinterpret_cast<float4*>(lds + (e / P4) * lds_stride + 4 * (e % P4)) = make_float4(v[i].x * f, v[i].y * f, v[i].z * f, v[i].w * f);
-        }
-    }
-};
-
 // U[idx, head] = sum_j e^(c_j - max c) k_j v_j^T [dk, dv], N[idx, head] the same sum of k_j, scal[idx, head] =
 // (F of the whole chunk, max c).  Grid (heads, chunks, blocks of 64 value channels); a wave takes rows of 16 x 16 tiles.
 // KQ: dk <= 4 KQ.  LDS: k [64][4 KQ + 4] (weighted), v [64][68], weights [64].  A matrix instruction sums 4 keys: lane
@@ -270,7 +202,7 @@ __global__ __launch_bounds__(256) void memory_sums_kernel(
     extern __shared__ __attribute__((aligned(16))) float mem_lds[];
     const int head = blockIdx.x, idx = blockIdx.y, vb = blockIdx.z * 64, tid = threadIdx.x;
     int item, chunk;
-    if (!memory_find_chunk(idx, item_len, item_slot, num_items, item, chunk)) return;
+    if (!find_chunk(idx, item_len, item_slot, num_items, item, chunk)) return;
     const int n = min(kMemChunk, item_len[item] - chunk * kMemChunk);
     const int64_t row0 = (int64_t)item_tok_off[item] + (int64_t)chunk * kMemChunk;
     const float* p = proj + row0 * stride;
@@ -406,7 +338,7 @@ __global__ __launch_bounds__(256) void memory_out_kernel(
     using L = MemoryOutLds<KQ, NV>;
     const int head = blockIdx.x, idx = blockIdx.y, tid = threadIdx.x;
     int item, chunk;
-    if (!memory_find_chunk(idx, item_len, item_slot, num_items, item, chunk)) return;
+    if (!find_chunk(idx, item_len, item_slot, num_items, item, chunk)) return;
     const int n = min(kMemChunk, item_len[item] - chunk * kMemChunk);
     const int64_t row0 = (int64_t)item_tok_off[item] + (int64_t)chunk * kMemChunk;
     const float* p = proj + row0 * stride;

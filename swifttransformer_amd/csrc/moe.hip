@@ -2,7 +2,7 @@
 // `experts` small gated feed-forward layers.
 //
 // Everything stays on the device and has a fixed launch shape, so a step can be recorded:
-//   route    per token the `top` best experts and their weights (four rules, see st_moe_route);
+//   route    per token the `top` best experts and their weights (five rules, see st_moe_route);
 //   align    the (token, choice) pairs sorted by expert into tiles of 16, 64 or 128 places, a tile
 //            holding pairs of one expert only (places left over are marked -1);
 //   up       per tile and 64 inner features: both input products on the matrix cores, rows
@@ -10,20 +10,19 @@
 //            without a gate: one product and the exact GELU);
 //   down     per tile and 64 output features: the output product; with one expert a token the
 //            result goes straight into the residual stream, otherwise to a row per pair that
-//   combine  sums in the order of the token's choices.
+//   combine  sums in the order of the token's choices.  Router outputs past the experts stand for identity
+//            experts: a choice of one has no place in the tiles, and its result is the token's own vector.
 // A wave computes 16 x 16 blocks of results with operands read straight from memory in the
 // matrix instruction's own layout (16 bytes a lane and step): with 16 rows a tile the products
 // are bound by the stream of expert weights, which every tile reads once.
 #include "api.h"
 #include "common.h"
 #include "activation.h"
+#include "fragment.h"
 
 #include <type_traits>
 
 namespace st {
-
-typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
-typedef float floatx4 __attribute__((ext_vector_type(4)));
 
 template <int N> using Steps = std::integral_constant<int, N>;
 constexpr int kRows = 16;            // rows of one matrix-instruction block
@@ -31,19 +30,19 @@ constexpr int kMaxTop = 16;
 
 __global__ __launch_bounds__(256) void moe_route_kernel(
     int* __restrict__ ids, float* __restrict__ weights, const float* __restrict__ logits,
-    const int* __restrict__ token_item, const float* __restrict__ correction, float scale, int num_tokens, int experts,
-    int top, int mode, int groups, int keep, int stage) {
+    int logit_stride, const int* __restrict__ token_item, const float* __restrict__ correction, float scale, int num_tokens,
+    int experts, int top, int mode, int groups, int keep, int stage) {
     // The rows of the workgroup's tokens go to LDS first, read side by side (a thread that walked its own row in
     // memory would wait for every logit by itself, several times over); rows are experts + 1 floats apart.
     extern __shared__ float s_z[];
     const int t0 = blockIdx.x * blockDim.x, t = t0 + threadIdx.x;
     if (stage) {
         const int n = min((int)blockDim.x, num_tokens - t0);
-        const float* src = logits + (int64_t)t0 * experts;
+        const float* src = logits + (int64_t)t0 * logit_stride;
         for (int i = threadIdx.x; i < n * experts; i += blockDim.x) {
             const int r = i / experts;
             // (mode 3 chooses by the sigmoid of a logit plus the expert's correction: formed here, side by side)
-            const float z = src[i];
+            const float z = src[(int64_t)r * logit_stride + (i - r * experts)];
             s_z[r * (experts + 1) + (i - r * experts)] = mode == 3 ? 1.f / (1.f + expf(-z)) + correction[i - r * experts] : z;
         }
         __syncthreads();
@@ -53,7 +52,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
         for (int j = 0; j < top; ++j) { ids[(int64_t)t * top + j] = -1; weights[(int64_t)t * top + j] = 0.f; }
         return;
     }
-    const float* z = stage ? s_z + threadIdx.x * (experts + 1) : logits + (int64_t)t * experts;
+    const float* z = stage ? s_z + threadIdx.x * (experts + 1) : logits + (int64_t)t * logit_stride;
     // mode 2: only the experts of the `keep` groups (of `groups` equal groups of neighbours) whose largest
     // logit is largest can be chosen; bit g of `open` says that group g is one of them
     uint64_t open = ~0ull;
@@ -72,18 +71,24 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
             open |= 1ull << best;
         }
     }
-    // mode 2: the weights are the chosen experts' shares of the softmax over all experts, as they are
+    // modes 2 and 4: the weights are the chosen experts' shares of the softmax over all experts, as they are
     float m_all = 0.f, inv_sum = 1.f;
-    if (mode == 2) {
+    if (mode == 2 || mode == 4) {
         m_all = z[0];
         for (int e = 1; e < experts; ++e) m_all = fmaxf(m_all, z[e]);
         float sum = 0.f;
         for (int e = 0; e < experts; ++e) sum += expf(z[e] - m_all);
         inv_sum = 1.f / sum;
     }
-    // mode 3: what an expert is chosen by, where it was not staged
+    // mode 4: the share plus the expert's correction chooses; staged, it takes the logit's place in this thread's own row
+    if (mode == 4 && stage) {
+        float* own = s_z + threadIdx.x * (experts + 1);
+        for (int e = 0; e < experts; ++e) own[e] = expf(own[e] - m_all) * inv_sum + correction[e];
+    }
+    // modes 3 and 4: what an expert is chosen by, where it was not staged
     auto choice = [&](int e) {
-        return mode == 3 && !stage ? 1.f / (1.f + expf(-z[e])) + correction[e] : z[e];
+        if (stage || mode < 3) return z[e];
+        return (mode == 3 ? 1.f / (1.f + expf(-z[e])) : expf(z[e] - m_all) * inv_sum) + correction[e];
     };
     auto weight_of = [&](float v) { return mode == 0 ? 1.f / (1.f + expf(-v)) : mode == 2 ? expf(v - m_all) * inv_sum : v; };
     if (experts <= 64) {
@@ -132,13 +137,17 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     } else if (mode == 3) {
         // the chosen experts' sigmoids, without the correction, over their sum
         float* w = weights + (int64_t)t * top;
-        const float* raw = logits + (int64_t)t * experts;
+        const float* raw = logits + (int64_t)t * logit_stride;
         float sum = 0.f;
         for (int j = 0; j < top; ++j) {
             w[j] = 1.f / (1.f + expf(-raw[ids[(int64_t)t * top + j]]));
             sum += w[j];
         }
         for (int j = 0; j < top; ++j) w[j] = w[j] / (sum + 1e-20f) * scale;
+    } else if (mode == 4) {
+        // the shares themselves, without the correction
+        const float* raw = logits + (int64_t)t * logit_stride;
+        for (int j = 0; j < top; ++j) weights[(int64_t)t * top + j] = expf(raw[ids[(int64_t)t * top + j]] - m_all) * inv_sum;
     }
 }
 
@@ -156,8 +165,8 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(
     for (int i = tid; i < capacity / kTile; i += 1024) tile_expert[i] = -1;
     __syncthreads();
     for (int p = tid; p < num_pairs; p += 1024) {
-        const int e = ids[p];
-        if (e >= 0) atomicAdd(&count[e], 1);
+        const int e = ids[p];                          // (an identity expert has no tiles)
+        if (e >= 0 && e < experts) atomicAdd(&count[e], 1);
     }
     __syncthreads();
     if (tid == 0) {
@@ -177,59 +186,13 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(
     for (int p = tid; p < num_pairs; p += 1024) {
         const int e = ids[p];
         int place = -1;
-        if (e >= 0) {
+        if (e >= 0 && e < experts) {
             place = atomicAdd(&count[e], 1);
             sorted[place] = p;
         }
         place_of_pair[p] = place;
     }
 }
-
-// ---- operands in the matrix instructions' layout: lane (r16, g) holds, of row r16, the elements
-// k0 + 8g .. 8g+7 (bfloat16, one product of depth 32) or k0 + 4g .. 4g+3 (float, four products
-// of depth 4, the u-th taking element u of every lane).
-template <typename T> struct Frag;
-template <> struct Frag<bf16_t> {
-    static constexpr int kDepth = 32, kLane = 8;
-    bf16x8 v;
-    __device__ inline void load_whole(const bf16_t* p) { v = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(p)); }
-    __device__ inline void load(const bf16_t* row, int k, int K, bool ok, bool vec) {
-        if (ok && vec && k + 8 <= K) {
-            v = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(row + k));
-        } else {
-            uint16_t e[8];
-#pragma unroll
-            for (int i = 0; i < 8; ++i) e[i] = (ok && k + i < K) ? row[k + i].bits : (uint16_t)0;
-            v = __builtin_bit_cast(bf16x8, make_uint4(e[0] | ((uint32_t)e[1] << 16), e[2] | ((uint32_t)e[3] << 16),
-                                                      e[4] | ((uint32_t)e[5] << 16), e[6] | ((uint32_t)e[7] << 16)));
-        }
-    }
-    __device__ static inline floatx4 mma(const Frag& a, const Frag& b, floatx4 c) {
-        return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, c, 0, 0, 0);
-    }
-};
-template <> struct Frag<float> {
-    static constexpr int kDepth = 16, kLane = 4;
-    float v[4];
-    __device__ inline void load_whole(const float* p) {
-        const float4 x = *reinterpret_cast<const float4*>(p);
-        v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w;
-    }
-    __device__ inline void load(const float* row, int k, int K, bool ok, bool vec) {
-        if (ok && vec && k + 4 <= K) {
-            const float4 x = *reinterpret_cast<const float4*>(row + k);
-            v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w;
-        } else {
-#pragma unroll
-            for (int i = 0; i < 4; ++i) v[i] = (ok && k + i < K) ? row[k + i] : 0.f;
-        }
-    }
-    __device__ static inline floatx4 mma(const Frag& a, const Frag& b, floatx4 c) {
-#pragma unroll
-        for (int u = 0; u < 4; ++u) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.v[u], b.v[u], c, 0, 0, 0);
-        return c;
-    }
-};
 
 // ---- few rows an expert: tiles of 16 places, where only the weights' stream counts.  A workgroup takes 16 features; its
 // four waves share the depth, so that a wave's part is one or a few batches of loads that are all on their way at once and
@@ -324,7 +287,7 @@ __global__ __launch_bounds__(256) void moe_up_few_kernel(
         const float gv = sum[MATS - 1];
         out = gv / (1.f + expf(-gv)) * sum[0];
     } else if (p >= 0) {
-        const float s = weights[p];
+        const float s = style == 0 ? weights[p] : 1.f;
         const float gv = fminf(s * sum[MATS - 1], limit);
         const float uv = fminf(fmaxf(s * sum[0], -limit), limit);
         out = gv / (1.f + expf(-1.702f * gv)) * (uv + 1.f);
@@ -442,7 +405,7 @@ __global__ __launch_bounds__(256) void moe_up_kernel(
                 const float gv = cg[b][r];
                 out = gv / (1.f + expf(-gv)) * cu[b][r];
             } else if (p >= 0) {
-                const float s = weights[p];
+                const float s = style == 0 ? weights[p] : 1.f;
                 const float gv = fminf(s * cg[b][r], limit);
                 const float uv = fminf(fmaxf(s * cu[b][r], -limit), limit);
                 out = gv / (1.f + expf(-1.702f * gv)) * (uv + 1.f);
@@ -616,7 +579,7 @@ __global__ __launch_bounds__(256) void moe_tiled_kernel(
         const int place = base + wm * 64 + j * 32 + l32;
         const int p = sorted[place];
         if (UP) {
-            const float s = p >= 0 && style == 0 ? weights[p] : 0.f;
+            const float s = p >= 0 && style == 0 ? weights[p] : 1.f;
 #pragma unroll
             for (int q4 = 0; q4 < 4; ++q4) {
                 const int f = n0 + wn * 32 + 8 * q4 + 4 * lh;
@@ -675,18 +638,20 @@ __global__ __launch_bounds__(256) void moe_tiled_kernel(
     }
 }
 
-// V columns a thread and turn (4: 16-byte accesses)
-template <int V>
+// V columns a thread and turn (4: 16-byte accesses).  x (or null): the tokens' own vectors, the results of the identity
+// experts, whose numbers are `experts` and above.
+template <typename T, int V>
 __global__ __launch_bounds__(256) void moe_combine_kernel(
     float* out, const float* residual, const float* __restrict__ pair_out,
-    const int* __restrict__ place_of_pair, const float* __restrict__ weights, int top, int width, float out_scale) {
+    const int* __restrict__ place_of_pair, const float* __restrict__ weights, const int* __restrict__ ids,
+    const T* __restrict__ x, int experts, int top, int width, float out_scale) {
     const int t = blockIdx.x;
     for (int n = threadIdx.x * V; n < width; n += 256 * V) {
-        float sum[V], base[V];
+        float sum[V], base[V], own[V];
         bool any = false;
         const int64_t at = (int64_t)t * width + n;
 #pragma unroll
-        for (int v = 0; v < V; ++v) { sum[v] = 0.f; base[v] = 0.f; }
+        for (int v = 0; v < V; ++v) { sum[v] = 0.f; base[v] = 0.f; own[v] = 0.f; }
         if (residual) {
             if (V == 4) {
                 const float4 r = *reinterpret_cast<const float4*>(residual + at);
@@ -695,21 +660,26 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(
                 base[0] = residual[at];
             }
         }
+        if (x) {
+#pragma unroll
+            for (int v = 0; v < V; ++v) own[v] = Elem<T>::load(x + at + v);
+        }
 #pragma unroll 2
         for (int j = 0; j < top; ++j) {
             const int place = place_of_pair[(int64_t)t * top + j];
             const float w = weights ? weights[(int64_t)t * top + j] : 1.f;
+            const bool identity = x && ids[(int64_t)t * top + j] >= experts;
             const float* src = pair_out + (int64_t)max(place, 0) * width + n;
-            float x[V];
+            float r[V];
             if (V == 4) {
-                const float4 r = *reinterpret_cast<const float4*>(src);
-                x[0] = r.x; x[1 % V] = r.y; x[2 % V] = r.z; x[3 % V] = r.w;
+                const float4 q = *reinterpret_cast<const float4*>(src);
+                r[0] = q.x; r[1 % V] = q.y; r[2 % V] = q.z; r[3 % V] = q.w;
             } else {
-                x[0] = src[0];
+                r[0] = src[0];
             }
-            if (place >= 0) {
+            if (place >= 0 || identity) {
 #pragma unroll
-                for (int v = 0; v < V; ++v) sum[v] = fmaf(w, x[v], sum[v]);
+                for (int v = 0; v < V; ++v) sum[v] = fmaf(w, identity ? own[v] : r[v], sum[v]);
                 any = true;
             }
         }
@@ -725,12 +695,13 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(
 
 using namespace st;
 
-extern "C" int st_moe_route(int* ids, float* weights, const float* logits, const int* token_item, const float* correction,
-                            float scale, int num_tokens, int experts, int top, int mode, int groups, int keep,
+extern "C" int st_moe_route(int* ids, float* weights, const float* logits, int logit_stride, const int* token_item,
+                            const float* correction, float scale, int num_tokens, int experts, int top, int mode, int groups, int keep,
                             hipStream_t stream) {
-    ST_CHECK(mode >= 0 && mode <= 3, "moe_route: mode 0 (sigmoid of each), 1 (softmax over the chosen), 2 (softmax "
-             "over all, the choice within the best groups) or 3 (sigmoids over their sum, a corrected choice)");
-    ST_CHECK(mode != 3 || correction, "moe_route: mode 3 chooses by corrected scores");
+    ST_CHECK(mode >= 0 && mode <= 4, "moe_route: mode 0 (sigmoid of each), 1 (softmax over the chosen), 2 (softmax "
+             "over all, the choice within the best groups), 3 (sigmoids over their sum, a corrected choice) or 4 (softmax over "
+             "all, a corrected choice)");
+    ST_CHECK(mode < 3 || correction, "moe_route: modes 3 and 4 choose by corrected scores");
     if (mode != 2) groups = keep = 1;
     ST_CHECK(groups >= 1 && groups <= 64 && experts % groups == 0 && keep >= 1 && keep <= groups,
              "moe_route: %d experts in %d groups of which %d are kept (up to 64 equal groups)", experts, groups, keep);
@@ -739,14 +710,14 @@ extern "C" int st_moe_route(int* ids, float* weights, const float* logits, const
     ST_CHECK(num_tokens >= 0 && experts > 0, "moe_route: bad sizes");
     ST_CHECK(top >= 1 && top <= kMaxTop && top <= experts, "moe_route: 1 to %d experts a token (of %d), not %d",
              kMaxTop, experts, top);
-    ST_CHECK(ids && weights && logits, "moe_route: null operand");
+    ST_CHECK(ids && weights && logits && logit_stride >= experts, "moe_route: null operand or short rows");
     if (num_tokens == 0) return 0;
     // workgroups of as many tokens as have their rows side by side in 48 KB of LDS (256, 64, or none staged)
     const size_t row = (size_t)(experts + 1) * sizeof(float);
     const int threads = 256 * row <= 48 * 1024 ? 256 : 64;
     const int stage = threads * row <= 48 * 1024;
     moe_route_kernel<<<(num_tokens + threads - 1) / threads, threads, stage ? threads * row : 0, stream>>>(
-        ids, weights, logits, token_item, correction, scale, num_tokens, experts, top, mode, groups, keep, stage);
+        ids, weights, logits, logit_stride, token_item, correction, scale, num_tokens, experts, top, mode, groups, keep, stage);
     ST_LAUNCH_CHECK("moe_route");
     return 0;
 }
@@ -775,7 +746,8 @@ extern "C" int st_moe_up(void* y, const void* x, const void* w_gate, const void*
                          const int* tile_expert, const float* weights, int capacity, int tile, int top, int width,
                          int inner, float limit, int style, int dtype, hipStream_t stream) {
     const int kTile = tile;
-    ST_CHECK(style >= 0 && style <= 2, "moe_up: style 0 (weighted, clamped inputs), 1 (plain gated unit) or 2 (no gate, GELU)");
+    ST_CHECK(style >= 0 && style <= 3, "moe_up: style 0 (weighted, clamped inputs), 1 (plain gated unit), 2 (no gate, GELU) or 3 "
+             "(clamped inputs, no weight)");
     if (style == 2) w_gate = w_up;
     ST_CHECK(tile == 16 || tile == 64 || tile == 128, "moe_up: tiles of 16, 64 or 128 places, not %d", tile);
     ST_CHECK(capacity > 0 && capacity % kTile == 0 && top >= 1 && width > 0 && inner > 0, "moe_up: bad sizes");
@@ -865,17 +837,22 @@ extern "C" int st_moe_down(float* out, const float* residual, float* pair_out, c
     return 0;
 }
 
+// ids and x (both or neither): a choice of `experts` or above is an identity expert, whose result is the token's row of x
+// [tokens, width] in the storage type.
 extern "C" int st_moe_combine(float* out, const float* residual, const float* pair_out, const int* place_of_pair,
-                              const float* weights, int num_tokens, int top, int width, float out_scale,
-                              hipStream_t stream) {
+                              const float* weights, const int* ids, const void* x, int experts, int num_tokens, int top,
+                              int width, float out_scale, int dtype, hipStream_t stream) {
     ST_CHECK(num_tokens >= 0 && top >= 1 && width > 0, "moe_combine: bad sizes");
-    ST_CHECK(out && pair_out && place_of_pair, "moe_combine: null operand");
+    ST_CHECK(out && pair_out && place_of_pair && (!x || ids), "moe_combine: null operand");
+    ST_CHECK(dtype == kF32 || dtype == kBF16, "moe_combine: unknown dtype %d", dtype);
     if (num_tokens == 0) return 0;
     const bool vec = width % 4 == 0 && (((uintptr_t)out | (uintptr_t)residual | (uintptr_t)pair_out) & 15) == 0;
-    if (vec)
-        moe_combine_kernel<4><<<num_tokens, 256, 0, stream>>>(out, residual, pair_out, place_of_pair, weights, top, width, out_scale);
-    else
-        moe_combine_kernel<1><<<num_tokens, 256, 0, stream>>>(out, residual, pair_out, place_of_pair, weights, top, width, out_scale);
+#define ST_MC(T, V)                                                                                                    \
+    moe_combine_kernel<T, V><<<num_tokens, 256, 0, stream>>>(out, residual, pair_out, place_of_pair, weights, ids, (const T*)x, \
+                                                             experts, top, width, out_scale)
+    if (dtype == kF32) { if (vec) ST_MC(float, 4); else ST_MC(float, 1); }
+    else { if (vec) ST_MC(bf16_t, 4); else ST_MC(bf16_t, 1); }
+#undef ST_MC
     ST_LAUNCH_CHECK("moe_combine");
     return 0;
 }

@@ -10,6 +10,7 @@ from . import zimorax  # noqa: F401  (registers Zimorax)
 from . import gisedra  # noqa: F401  (registers Gisedra)
 from . import pupalix  # noqa: F401  (registers Pupalix)
 from . import fiterax  # noqa: F401  (registers Fiterax)
+from . import fefozen  # noqa: F401  (registers Fefozen)
 from .opt import build_opt_spec
 
 __all__ = ["DecoderModel", "build_opt_spec", "build_model", "load_model", "random_model"]

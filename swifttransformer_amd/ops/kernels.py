@@ -92,13 +92,34 @@ def _lib():
                                            _c_f, _c_int, _c_p]
         lib.st_latent_write.argtypes = [_c_p, _c_i64, _c_p, _c_i64, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int,
                                         _c_int, _c_int, _c_f, _c_int, _c_p, _c_f, _c_int, _c_p]
-        lib.st_moe_route.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_p, _c_f, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_p]
+        lib.st_moe_route.argtypes = [_c_p, _c_p, _c_p, _c_int, _c_p, _c_p, _c_f, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_p]
         lib.st_moe_align.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_p]
         lib.st_moe_up.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_int,
                                   _c_f, _c_int, _c_int, _c_p]
         lib.st_moe_down.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_int,
                                     _c_f, _c_int, _c_p]
-        lib.st_moe_combine.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_f, _c_p]
+        lib.st_moe_combine.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_f, _c_int,
+                                       _c_p]
+        lib.st_latent_inputs.argtypes = [_c_p, _c_int, _c_p, _c_int, _c_p, _c_i64, _c_p, _c_int, _c_int, _c_int, _c_p, _c_int,
+                                         _c_f, _c_int, _c_p, _c_i64, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_f, _c_int,
+                                         _c_p]
+        lib.st_latent_tiles.argtypes = [_c_p, _c_p, _c_i64, _c_p, _c_i64, _c_p, _c_p, _c_int, _c_p, _c_p, _c_p, _c_p, _c_p,
+                                        _c_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f, _c_f, _c_int,
+                                        _c_int, _c_p]
+        lib.st_latent_rows.argtypes = [_c_p, _c_p, _c_p, _c_i64, _c_p, _c_i64, _c_p, _c_p, _c_p, _c_int, _c_int, _c_p, _c_p,
+                                       _c_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f, _c_f, _c_int,
+                                       _c_int, _c_p]
+        lib.st_latent_merge.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_p]
+        lib.st_latent_up.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_int, _c_p, _c_p, _c_i64, _c_p, _c_int, _c_int, _c_int, _c_int,
+                                     _c_int, _c_p]
+        lib.st_delta_slot.restype = _c_i64
+        lib.st_delta_slot.argtypes = [_c_int] * 5
+        lib.st_delta_step.argtypes = [_c_p, _c_p, _c_i64, _c_p, _c_i64, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_int,
+                                      _c_int, _c_int, _c_int, _c_int, _c_int, _c_f, _c_f, _c_f, _c_int, _c_p]
+        lib.st_delta_chunks.argtypes = [_c_p, _c_p, _c_i64, _c_p, _c_i64, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p,
+                                        _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_f, _c_f, _c_f, _c_p, _c_p,
+                                        _c_p, _c_p, _c_p, _c_p, _c_p, _c_i64, _c_int, _c_p]
+        lib.st_rms_onto.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int, _c_f, _c_f, _c_int, _c_p]
         lib.st_dynamic_tanh.argtypes = [_c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_p, _c_int, _c_int,
                                         _c_int, _c_p]
         lib.st_unit_add.argtypes = [_c_p, _c_p, _c_p, _c_int, _c_int, _c_f, _c_p]
@@ -1280,7 +1301,8 @@ def routed_experts(x: torch.Tensor, logits: torch.Tensor, w_gate: Optional[torch
                    w_down: torch.Tensor, residual: Optional[torch.Tensor], *, top: int, limit: float = 0.0,
                    out_scale: float = 1.0, token_item: Optional[torch.Tensor] = None,
                    style: str = "scaled_input", groups: int = 1, keep: int = 1,
-                   correction: Optional[torch.Tensor] = None, scale: float = 1.0) -> torch.Tensor:
+                   correction: Optional[torch.Tensor] = None, scale: float = 1.0, identity: int = 0,
+                   clamped: bool = False) -> torch.Tensor:
     """residual <- residual + out_scale * sum over a row's ``top`` best experts e (by ``logits``) of
     Wd[e] y with y = g * sigmoid(1.702 g) * (u + 1), g = min(s * Wg[e] x, limit),
     u = clamp(s * Wu[e] x, -limit, limit), s = sigmoid(logit of e).  In place on ``residual``
@@ -1294,27 +1316,40 @@ def routed_experts(x: torch.Tensor, logits: torch.Tensor, w_gate: Optional[torch
     a group ranking by its largest logit.
     ``style`` "sigmoid_output": a row's experts are those with the largest sigmoid(logit) + ``correction`` (float
     [experts]), weighted by scale * sigmoid(logit) / (the chosen sigmoids' sum + 1e-20).
+    ``style`` "softmax_corrected": those with the largest share of the softmax over all logits + ``correction``, weighted by
+    the shares as they are.
+
+    ``identity`` > 0 (styles with weights on the results): so many more logits (and corrections) behind the experts' stand
+    for identity experts, whose result is x itself.  ``clamped``: the experts of these styles are the first style's gated
+    unit with ``limit`` (and s = 1) instead of the plain one.
 
     ``w_gate`` None (not in the first style): experts without a gate, Wd[e] gelu(Wu[e] x), the exact GELU.
 
-    x: [T, width]; logits: float [T, experts]; w_gate, w_up: [experts, inner, width]; w_down:
+    x: [T, width]; logits: float [T, experts + identity] (rows may be longer and of any stride); w_gate, w_up: [experts, inner, width]; w_down:
     [experts, width, inner].  Rows whose ``token_item`` is negative are left as they are."""
     T, W = x.shape
     E, F, _ = w_up.shape
     _need(x, "x", w_up.dtype, (T, W))
-    _need(logits, "logits", torch.float32, (T, E))
+    outputs = E + int(identity)
+    _need(logits, "logits", torch.float32, (T, logits.shape[1]), contiguous=False)
+    if logits.shape[1] < outputs or logits.stride(1) != 1:
+        raise KernelError(f"logits: dense rows of {outputs}")
     if w_gate is not None:
         _need(w_gate, "w_gate", w_up.dtype, (E, F, W))
     _need(w_up, "w_up", None, (E, F, W))
     _need(w_down, "w_down", w_up.dtype, (E, W, F))
-    if style not in ("scaled_input", "softmax_output", "softmax_all", "sigmoid_output"):
+    if style not in ("scaled_input", "softmax_output", "softmax_all", "sigmoid_output", "softmax_corrected"):
         raise KernelError(f"routed_experts: unknown style {style!r}")
     on_output = style != "scaled_input"
-    mode = {"scaled_input": 0, "softmax_output": 1, "softmax_all": 2, "sigmoid_output": 3}[style]
+    mode = {"scaled_input": 0, "softmax_output": 1, "softmax_all": 2, "sigmoid_output": 3, "softmax_corrected": 4}[style]
     if w_gate is None and not on_output:
         raise KernelError("routed_experts: this style has gated experts")
-    if mode == 3:
-        _need(correction, "correction", torch.float32, (E,))
+    if identity and not on_output:
+        raise KernelError("routed_experts: identity experts go with weights on the results")
+    if clamped and (w_gate is None or not on_output):
+        raise KernelError("routed_experts: the clamped unit is a gated one, with weights on its result")
+    if mode >= 3:
+        _need(correction, "correction", torch.float32, (outputs,))
     if mode == 2 and (groups < 1 or E % groups or not 1 <= keep <= groups or top > keep * (E // groups)):
         raise KernelError(f"routed_experts: {top} of {E} experts in {groups} groups of which {keep} are kept")
     if residual is None and not on_output:
@@ -1332,18 +1367,18 @@ def routed_experts(x: torch.Tensor, logits: torch.Tensor, w_gate: Optional[torch
     place = empty((T * top,), torch.int32, dev)
     tile_expert = empty((cap // tile,), torch.int32, dev)
     y = empty((cap, F), x.dtype, dev)
-    _check(lib.st_moe_route(_ptr(ids), _ptr(wts), _ptr(logits), _ptr(token_item),
-                            _ptr(correction) if mode == 3 else None, float(scale), T, E, int(top), mode, int(groups), int(keep), st))
+    _check(lib.st_moe_route(_ptr(ids), _ptr(wts), _ptr(logits), logits.stride(0) if T > 1 else logits.shape[1], _ptr(token_item),
+                            _ptr(correction) if mode >= 3 else None, float(scale), T, outputs, int(top), mode, int(groups), int(keep), st))
     _check(lib.st_moe_align(_ptr(sorted_pairs), _ptr(place), _ptr(tile_expert), _ptr(ids), T * top, E, cap, tile, st))
     _check(lib.st_moe_up(_ptr(y), _ptr(x), _ptr(w_gate), _ptr(w_up), _ptr(sorted_pairs), _ptr(tile_expert),
-                         _ptr(wts), cap, tile, int(top), W, F, float(limit), 2 if w_gate is None else int(on_output), code, st))
+                         _ptr(wts), cap, tile, int(top), W, F, float(limit), 2 if w_gate is None else 3 if clamped else int(on_output), code, st))
     if on_output:
         out = residual if residual is not None else empty((T, W), torch.float32, dev)
         pair_out = empty((cap, W), torch.float32, dev)
         _check(lib.st_moe_down(None, None, _ptr(pair_out), _ptr(y), _ptr(w_down), _ptr(sorted_pairs),
                                _ptr(tile_expert), cap, tile, int(top), W, F, 1.0, code, st))
-        _check(lib.st_moe_combine(_ptr(out), _ptr(residual), _ptr(pair_out), _ptr(place), _ptr(wts), T, int(top), W,
-                                  float(out_scale), st))
+        _check(lib.st_moe_combine(_ptr(out), _ptr(residual), _ptr(pair_out), _ptr(place), _ptr(wts), _ptr(ids),
+                                  _ptr(x) if identity else None, E, T, int(top), W, float(out_scale), code, st))
         return out
     if top == 1:
         _check(lib.st_moe_down(_ptr(residual), _ptr(residual), None, _ptr(y), _ptr(w_down), _ptr(sorted_pairs),
@@ -1352,8 +1387,8 @@ def routed_experts(x: torch.Tensor, logits: torch.Tensor, w_gate: Optional[torch
         pair_out = empty((cap, W), torch.float32, dev)
         _check(lib.st_moe_down(None, None, _ptr(pair_out), _ptr(y), _ptr(w_down), _ptr(sorted_pairs),
                                _ptr(tile_expert), cap, tile, int(top), W, F, float(out_scale), code, st))
-        _check(lib.st_moe_combine(_ptr(residual), _ptr(residual), _ptr(pair_out), _ptr(place), None, T, int(top), W,
-                                  float(out_scale), st))
+        _check(lib.st_moe_combine(_ptr(residual), _ptr(residual), _ptr(pair_out), _ptr(place), None, None, None, E, T, int(top), W,
+                                  float(out_scale), code, st))
     return residual
 
 
@@ -1777,6 +1812,269 @@ def matrix_memory(proj: torch.Tensor, bias_i: torch.Tensor, bias_f: torch.Tensor
     _check(lib.st_memory_chunks(*head, T, heads, key_dim, value_dim, float(cap), q_scale, float(eps), _ptr(u), _ptr(n),
                                 _ptr(sc), _ptr(m), chunks, code, _stream()))
     return out
+
+
+# --------------------------------------------------------- gated delta rule
+def delta_row(heads: int, qk_heads: int, key_dim: int, value_dim: int) -> int:
+    """Floats of a row of ``delta_rule``'s input: q | k | v | gate | write strength | decay (logits)."""
+    return 2 * qk_heads * key_dim + 2 * heads * (value_dim + 1)
+
+
+def delta_slot(heads: int, qk_heads: int, key_dim: int, value_dim: int, taps: int) -> int:
+    """Floats of a request's state: a ring of the filter's last inputs [taps, channels] | S [heads, key_dim, value_dim],
+    each filled up to whole 16-byte pieces."""
+    ring = -(-taps * (2 * qk_heads * key_dim + heads * value_dim) // 4) * 4
+    return ring + -(-heads * key_dim * value_dim // 4) * 4
+
+
+def _d_delta(proj, taps_w, a_log, dt_bias, gain, state, ctx_arrays, heads, qk_heads, key_dim, value_dim, eps, unit_eps,
+             out_dtype, all_single=False):
+    T, B = proj.shape[0], ctx_arrays[3].shape[0]
+    es = torch.empty((), dtype=out_dtype).element_size()
+    return {"rows": T, "heads": heads, "key_dim": key_dim, "value_dim": value_dim, "items": B,
+            "flops": 6 * T * heads * key_dim * value_dim,
+            "bytes": T * (4 * delta_row(heads, qk_heads, key_dim, value_dim) + es * heads * value_dim) +
+                     8 * B * heads * key_dim * value_dim}
+
+
+@_timed("delta_rule", _d_delta)
+def delta_rule(proj: torch.Tensor, taps_w: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor, gain: torch.Tensor,
+               state: torch.Tensor, ctx_arrays, heads: int, qk_heads: int, key_dim: int, value_dim: int, eps: float,
+               unit_eps: float, out_dtype: torch.dtype, all_single: bool = False) -> torch.Tensor:
+    """Per item and head, from the slot's state and over the item's rows in order: q, k and v through a causal filter a
+    channel (``taps_w`` float [taps, channels], the last row meets the token itself) and SiLU, q and k at unit length
+    (``unit_eps`` under the root), q times key_dim^-1/2; S <- g S, u = b (v - S^T k), S <- S + k u^T, o = S^T q with
+    g = exp(-exp(a_log) softplus(decay logit + dt_bias)), b = sigmoid(strength logit); the result is o at unit root mean
+    square a head times ``gain`` [value_dim] times silu(gate), in ``out_dtype``.  The state is stored back.
+
+    proj: float rows (dense, any stride) that start with q | k | v | gate | strength | decay (``delta_row``); state: float
+    [slots, delta_slot].  ``ctx_arrays``: the batch's (token_item, positions, item_len, item_tok_off, item_slot).
+    ``all_single``: every item has one row (one kernel); otherwise products within chunks of rows and a carry between
+    chunks.  Rows of no item are left as they are."""
+    token_item, positions, item_len, item_tok_off, item_slot = ctx_arrays
+    T = proj.shape[0]
+    taps, C = taps_w.shape
+    _need(proj, "proj", torch.float32, (T, proj.shape[1]), contiguous=False)
+    if proj.stride(1) != 1 or proj.shape[1] < delta_row(heads, qk_heads, key_dim, value_dim):
+        raise KernelError("proj: dense rows that hold q, k, v, the gate and the gates of the recurrence")
+    if C != 2 * qk_heads * key_dim + heads * value_dim:
+        raise KernelError(f"delta_rule: filters for {C} channels")
+    _need(taps_w, "taps_w", torch.float32, (taps, C))
+    _need(a_log, "a_log", torch.float32, (heads,))
+    _need(dt_bias, "dt_bias", torch.float32, (heads,))
+    _need(gain, "gain", torch.float32, (value_dim,))
+    slot_stride = _slot_rows(state, "state", delta_slot(heads, qk_heads, key_dim, value_dim, taps))
+    B = item_slot.shape[0]
+    for name, t, n in (("token_item", token_item, T), ("positions", positions, T), ("item_len", item_len, B),
+                       ("item_tok_off", item_tok_off, B), ("item_slot", item_slot, B)):
+        _need(t, name, torch.int32, (n,))
+    lib, dev, code = _lib(), proj.device, dtype_code(out_dtype)
+    out = empty((T, heads * value_dim), out_dtype, dev)
+    stride = proj.stride(0) if T > 1 else proj.shape[1]
+    head = (_ptr(out), _ptr(proj), stride, _ptr(state), slot_stride, _ptr(taps_w), _ptr(a_log), _ptr(dt_bias), _ptr(gain))
+    sizes = (heads, qk_heads, key_dim, value_dim, taps, float(key_dim) ** -0.5, float(unit_eps), float(eps))
+    if all_single:
+        _check(lib.st_delta_step(*head, _ptr(positions), _ptr(item_len), _ptr(item_tok_off), _ptr(item_slot), B, *sizes, code,
+                                 _stream()))
+        return out
+    rows = int(lib.st_delta_chunk_rows())
+    chunks = T // rows + B
+    f = lambda *shape: empty(shape, torch.float32, dev)
+    scratch = (f(T, C), f(T, 2 * heads), f(chunks, heads, rows, value_dim), f(chunks, heads, rows, key_dim),
+               f(chunks, heads, key_dim, rows), f(chunks, heads), f(chunks, heads, key_dim, value_dim))
+    _check(lib.st_delta_chunks(*head, _ptr(token_item), _ptr(positions), _ptr(item_len), _ptr(item_tok_off), _ptr(item_slot), B, T,
+                               *sizes, *[_ptr(t) for t in scratch], chunks, code, _stream()))
+    return out
+
+
+# ------------------------------------- attention over a latent cache shared by all heads
+def latent_max_entry() -> int:
+    """The largest cached entry (a multiple of 16) that the latent attention kernels take."""
+    return int(_lib().st_latent_max_entry())
+
+
+class LatentShape:
+    """How a latent cache and its queries are laid out: ``entry`` dims a cached vector and query head, of which the first
+    ``out_dim`` make the result; pairs (rot_off + 2i, rot_off + 2i + 1) of a query turn by position * freq[i] (``freq``
+    float on the device, or None); ``sink`` float [heads] or None; ``window`` > 0: the last positions only."""
+
+    def __init__(self, heads: int, entry: int, out_dim: int, scale: float, rot_off: int = 0, freq: Optional[torch.Tensor] = None,
+                 rot_mult: float = 1.0, sink: Optional[torch.Tensor] = None, window: int = 0):
+        self.heads, self.entry, self.out_dim, self.scale = int(heads), int(entry), int(out_dim), float(scale)
+        self.rot_off, self.freq, self.rot_mult, self.sink, self.window = int(rot_off), freq, float(rot_mult), sink, int(window)
+
+
+def _latent_common(q, cache, block_table, sh: LatentShape):
+    pages, one, ps, entry = cache.shape
+    _need(cache, "cache", q.dtype, (pages, 1, ps, sh.entry), contiguous=False)
+    if cache.stride()[1:] != (ps * entry, entry, 1):
+        raise KernelError("latent attention: pages of one shared head must be contiguous")
+    _need(q, "q", None, (q.shape[0], sh.heads * sh.entry))
+    _need(block_table, "block_table", torch.int32)
+    if sh.sink is not None:
+        _need(sh.sink, "sink", torch.float32, (sh.heads,))
+    half = 0
+    if sh.freq is not None:
+        half = sh.freq.shape[0]
+        _need(sh.freq, "freq", torch.float32, (half,))
+    tail = (_ptr(block_table), _ptr(sh.sink), _ptr(sh.freq), block_table.shape[1], ps, sh.heads, sh.entry, sh.out_dim, sh.rot_off,
+            half, sh.rot_mult, sh.scale, sh.window, dtype_code(q.dtype), _stream())
+    return (_ptr(q), sh.heads * sh.entry, _ptr(cache), cache.stride(0)), tail
+
+
+@_timed("latent_inputs", lambda x, q_rank, q_width, gain_q, eps, cache=None, **k: {
+    "rows": x.shape[0], "width": q_rank + (k.get("rank", 0) + k.get("tail", 0)),
+    "bytes": x.shape[0] * (4 * (q_rank + k.get("rank", 0) + k.get("tail", 0)) +
+                           gain_q.element_size() // 2 * (q_width + (cache.shape[3] if cache is not None else 0)))})
+def latent_inputs(x: torch.Tensor, q_rank: int, q_width: int, gain_q: torch.Tensor, eps: float, cache: Optional[torch.Tensor] = None,
+                  *, dtype: torch.dtype, gain: Optional[torch.Tensor] = None, rank: int = 0, tail_off: int = 0, tail: int = 0,
+                  tail_freq: Optional[torch.Tensor] = None, tail_mult: float = 1.0, ctx_arrays=None) -> torch.Tensor:
+    """From float rows x (dense, any stride) q latent [q_rank] | latent [rank] | key part [tail]: returns the query latent at
+    unit root mean square times ``gain_q`` in ``dtype``, rows of q_width (zeros past q_rank); with ``cache`` [pages, 1,
+    page_size, entry], writes each token's entry: the latent at unit root mean square times ``gain``, the key part at
+    ``tail_off``, its pairs (2i, 2i + 1) turned by position * tail_freq[i] (cosine and sine times ``tail_mult``), zeros
+    elsewhere.  ``ctx_arrays``: (token_item, positions, block_table), with ``cache``."""
+    T = x.shape[0]
+    need = q_rank + (rank + tail if cache is not None else 0)
+    _need(x, "x", torch.float32, (T, x.shape[1]), contiguous=False)
+    if x.stride(1) != 1 or x.shape[1] < need:
+        raise KernelError("latent_inputs: dense rows that hold the latents and the key part")
+    _need(gain_q, "gain_q", torch.float32, (q_rank,))
+    cq = empty((T, q_width), dtype, x.device)
+    stride = x.stride(0) if T > 1 else x.shape[1]
+    if cache is None:
+        _check(_lib().st_latent_inputs(_ptr(cq), q_width, _ptr(gain_q), q_rank, None, 0, None, 0, 0, 0, None, 0, 1.0, 0, _ptr(x),
+                                       stride, None, None, None, 0, 0, T, float(eps), dtype_code(dtype), _stream()))
+        return cq
+    token_item, positions, block_table = ctx_arrays
+    pages, one, ps, entry = cache.shape
+    _need(cache, "cache", dtype, (pages, 1, ps, entry), contiguous=False)
+    if cache.stride()[1:] != (ps * entry, entry, 1):
+        raise KernelError("latent_inputs: pages of one shared head must be contiguous")
+    _need(gain, "gain", torch.float32, (rank,))
+    _need(token_item, "token_item", torch.int32, (T,))
+    _need(positions, "positions", torch.int32, (T,))
+    _need(block_table, "block_table", torch.int32)
+    half = 0
+    if tail_freq is not None:
+        half = tail_freq.shape[0]
+        _need(tail_freq, "tail_freq", torch.float32, (half,))
+    _check(_lib().st_latent_inputs(_ptr(cq), q_width, _ptr(gain_q), q_rank, _ptr(cache), cache.stride(0), _ptr(gain), rank,
+                                   int(tail_off), int(tail), _ptr(tail_freq), half, float(tail_mult), entry, _ptr(x), stride,
+                                   _ptr(token_item), _ptr(positions), _ptr(block_table), block_table.shape[1], ps, T, float(eps),
+                                   dtype_code(dtype), _stream()))
+    return cq
+
+
+def _d_latent_tiles(q, cache, tile_item, tile_q0, item_tok_off, item_start, item_len, block_table, sh, out):
+    return {"rows": q.shape[0], "heads": sh.heads, "kv_heads": 1, "head_dim": sh.entry, "value_dim": sh.out_dim,
+            "window": sh.window, "elem": q.element_size()}
+
+
+@_timed("latent_tiles", _d_latent_tiles)
+def latent_tiles(q: torch.Tensor, cache: torch.Tensor, tile_item: torch.Tensor, tile_q0: torch.Tensor, item_tok_off: torch.Tensor,
+                 item_start: torch.Tensor, item_len: torch.Tensor, block_table: torch.Tensor, sh: LatentShape,
+                 out: torch.Tensor) -> None:
+    """Attention of the items in the tile list (tiles of 64 tokens, as ``attention_prefill``'s) over a latent cache:
+    out [T, heads * out_dim] (of q's dtype) receives each head's weighted sum of the latents."""
+    head, tail = _latent_common(q, cache, block_table, sh)
+    n = tile_item.shape[0]
+    _need(tile_item, "tile_item", torch.int32, (n,))
+    _need(tile_q0, "tile_q0", torch.int32, (n,))
+    B = item_len.shape[0]
+    for name, t in (("item_tok_off", item_tok_off), ("item_start", item_start), ("item_len", item_len)):
+        _need(t, name, torch.int32, (B,))
+    _need(out, "out", q.dtype, (q.shape[0], sh.heads * sh.out_dim))
+    _check(_lib().st_latent_tiles(_ptr(out), *head, _ptr(tile_item), _ptr(tile_q0), n, _ptr(item_tok_off), _ptr(item_start),
+                                  _ptr(item_len), *tail))
+
+
+@_timed("latent_rows", lambda q, cache, token_item, positions, block_table, sh, num_splits=1, row_ids=None: {
+    "rows": row_ids.shape[0] if row_ids is not None else q.shape[0], "heads": sh.heads, "kv_heads": 1, "head_dim": sh.entry,
+    "value_dim": sh.out_dim, "window": sh.window, "splits": num_splits, "elem": q.element_size()})
+def latent_rows(q: torch.Tensor, cache: torch.Tensor, token_item: torch.Tensor, positions: torch.Tensor, block_table: torch.Tensor,
+                sh: LatentShape, num_splits: int = 1, row_ids: Optional[torch.Tensor] = None) -> SplitAttention:
+    """Attention of single rows (of the batch rows ``row_ids``, -1 skipped; all rows if None) over a latent cache, keys in
+    ``num_splits`` shares: the partial results [rows, heads, splits, out_dim], each normalised, with their log-sum-exps (a
+    sink is part of the first share)."""
+    head, tail = _latent_common(q, cache, block_table, sh)
+    T = q.shape[0]
+    n = row_ids.shape[0] if row_ids is not None else T
+    if row_ids is not None:
+        _need(row_ids, "row_ids", torch.int32, (n,))
+    _need(token_item, "token_item", torch.int32, (T,))
+    _need(positions, "positions", torch.int32, (T,))
+    part_o = empty((n, sh.heads, num_splits, sh.out_dim), torch.float32, q.device)
+    part_lse = empty((n, sh.heads, num_splits), torch.float32, q.device)
+    _check(_lib().st_latent_rows(_ptr(part_o), _ptr(part_lse), *head, _ptr(row_ids), _ptr(token_item), _ptr(positions), n,
+                                 int(num_splits), *tail))
+    return SplitAttention(part_o, part_lse)
+
+
+def latent_merge(part: SplitAttention, out: torch.Tensor, row_ids: Optional[torch.Tensor] = None) -> None:
+    """The shares of ``latent_rows`` merged into rows ``row_ids`` of out [T, heads * out_dim]."""
+    n, heads, splits, od = part.part_o.shape
+    _need(out, "out", None, (out.shape[0], heads * od))
+    _check(_lib().st_latent_merge(_ptr(out), _ptr(part.part_o), _ptr(part.part_lse), _ptr(row_ids), n, heads, od, splits,
+                                  dtype_code(out.dtype), _stream()))
+
+
+@_timed("latent_up", lambda o, w, gate=None, token_item=None: {
+    "rows": o.part_o.shape[0] if isinstance(o, SplitAttention) else o.shape[0], "heads": w.shape[0], "value_dim": w.shape[1],
+    "out_dim": w.shape[2], "flops": 2 * (o.part_o.shape[0] if isinstance(o, SplitAttention) else o.shape[0]) * w.numel(),
+    "bytes": w.numel() * w.element_size() +
+             (o.part_o.numel() * 4 if isinstance(o, SplitAttention) else o.numel() * o.element_size()) +
+             (o.part_o.shape[0] if isinstance(o, SplitAttention) else o.shape[0]) * w.shape[0] * w.shape[1] *
+             (w.element_size() + (4 if gate is not None else 0))})
+def latent_up(o, w: torch.Tensor, gate: Optional[torch.Tensor] = None, token_item: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """y [T, heads * value_dim] = W_h o_h a head (w [heads, value_dim, out_dim]) times the logistic function of ``gate``
+    (float [T, heads * value_dim], dense rows of any stride; None: no gate).  o: [T, heads * out_dim] of w's dtype, or
+    what ``latent_rows`` left for all rows of the batch (``token_item``: rows of no item are left as they are)."""
+    heads, vd, od = w.shape
+    _need(w, "w", None, (heads, vd, od))
+    split = isinstance(o, SplitAttention)
+    T = o.part_o.shape[0] if split else o.shape[0]
+    dev = o.part_o.device if split else o.device
+    if split:
+        if tuple(o.part_o.shape[1:2] + o.part_o.shape[3:]) != (heads, od) or token_item is None:
+            raise KernelError("latent_up: the partial results do not fit the matrices, or token_item is missing")
+        _need(token_item, "token_item", torch.int32, (T,))
+    else:
+        _need(o, "o", w.dtype, (T, heads * od))
+    stride = 0
+    if gate is not None:
+        _need(gate, "gate", torch.float32, (T, heads * vd), contiguous=False)
+        if gate.stride(1) != 1:
+            raise KernelError("gate: rows must be dense")
+        stride = gate.stride(0) if T > 1 else heads * vd
+    y = empty((T, heads * vd), w.dtype, dev)
+    _check(_lib().st_latent_up(_ptr(y), None if split else _ptr(o), _ptr(o.part_o) if split else None,
+                               _ptr(o.part_lse) if split else None, o.part_o.shape[2] if split else 1, _ptr(w), _ptr(gate), stride,
+                               _ptr(token_item) if split else None, T, heads, vd, od, dtype_code(w.dtype), _stream()))
+    return y
+
+
+# ------------------- a branch's result into the residual stream through a norm
+@_timed("rms_onto", lambda y, x, gain, eps, then=None, out_dtype=None: {
+    "rows": y.shape[0], "width": y.shape[1],
+    "bytes": y.numel() * (12 + (torch.empty((), dtype=out_dtype).element_size() if then is not None else 0))})
+def rms_onto(y: torch.Tensor, x: torch.Tensor, gain: torch.Tensor, eps: float, then: Optional[tuple] = None,
+             out_dtype: Optional[torch.dtype] = None):
+    """x + y / sqrt(mean(y^2) + eps) * gain row by row, a new float tensor; with ``then`` = (gain2, eps2): (that sum, its own
+    norm with gain2 and eps2 in ``out_dtype``), made in the same pass."""
+    T, W = y.shape
+    _need(y, "y", torch.float32, (T, W))
+    _need(x, "x", torch.float32, (T, W))
+    _need(gain, "gain", torch.float32, (W,))
+    out = empty((T, W), torch.float32, y.device)
+    if then is None:
+        _check(_lib().st_rms_onto(_ptr(out), None, _ptr(y), _ptr(x), _ptr(gain), None, T, W, float(eps), 0.0, F32, _stream()))
+        return out
+    _need(then[0], "gain2", torch.float32, (W,))
+    h = empty((T, W), out_dtype, y.device)
+    _check(_lib().st_rms_onto(_ptr(out), _ptr(h), _ptr(y), _ptr(x), _ptr(gain), _ptr(then[0]), T, W, float(eps), float(then[1]),
+                              dtype_code(out_dtype), _stream()))
+    return out, h
 
 
 def probe_read(src: torch.Tensor, sink: torch.Tensor, workgroups: int, pattern: int = 0) -> None:

@@ -38,7 +38,8 @@ HIPCC_FLAGS = [
 # accumulation registers
 FILE_FLAGS = {"attention_prefill.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
               "attention_prefill_dma.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
-              "attention_prefill_f32.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"]}
+              "attention_prefill_f32.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
+              "latent_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"]}
 # the vendor's matrix-product library backs the large bfloat16 products (csrc/gemm_library.hip)
 LINK_LIBS = ["-lhipblaslt"]
 

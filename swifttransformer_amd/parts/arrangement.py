@@ -8,7 +8,8 @@ post-norm (the reference refuses it, gpt.cc:238-240):
     r = N1(x + Mix(x)); x' = N2(r + FFN(r))
 sandwich (norms before and after each sublayer; the reference has no such block):
     r = x + N1b(Mix(N1(x))); s = r + N2b(FFN(N2(r))); x' = s + Side(s, token)
-    (the feed-forward and the side input are optional)
+    (the feed-forward and the side input are optional; where the norms allow, a norm after a branch, the sum into the
+    stream and the norm before the next branch, the next layer's included, are one pass)
 hyper-connections (several copies of the stream; the reference has no such block):
     u = sum_s a1[s] x_s;  y = Mix(N1(u));  x_t <- sum_s M1[s, t] x_s + b1[t] y   (all t at once)
     and the same with a2, M2, b2 around the feed-forward, which is optional
@@ -76,9 +77,14 @@ class PostNorm(Part):
 
 
 class Sandwich(Part):
-    """params: feed_forward (bool, default True).  The mixer and the feed-forward are asked for their
+    """params: feed_forward (bool, default True).  names (a layer without feed-forward): unused_norm, unused_out_norm, norms
+    that a file may hold all the same.  The mixer and the feed-forward are asked for their
     results alone (``residual32`` None, which they must allow: ``raw_output_ok``); the norm after each adds
-    its result to the stream (``forward_onto``).  A ``side_input`` part of the layer acts on the stream last."""
+    its result to the stream (``forward_onto``).  A ``side_input`` part of the layer acts on the stream last; without one,
+    the last norm also makes the first norm of the layer ``then`` that runs next, where the two chain, and leaves it with
+    the step's context (``reads_ahead``)."""
+
+    reads_ahead = True
 
     def __init__(self, spec, hidden_size, dtype):
         super().__init__(spec, hidden_size, dtype)
@@ -86,11 +92,20 @@ class Sandwich(Part):
         self.needs = (("mixer_norm", "mixer_out_norm", "ffn_norm", "feed_forward", "ffn_out_norm") if self.has_ffn
                       else ("mixer_norm", "mixer_out_norm"))
 
-    def forward(self, x32: torch.Tensor, layer, ctx, cache, write: bool = True) -> torch.Tensor:
+    def tensor_specs(self) -> List[TensorSpec]:
+        # a layer without feed-forward: a file may still hold its norms; they are not read
+        return [TensorSpec(self.name(n), (self.hidden_size,), "vector", optional=True)
+                for n in ("unused_norm", "unused_out_norm") if n in self.spec.names]
+
+    def forward(self, x32: torch.Tensor, layer, ctx, cache, write: bool = True, then=None) -> torch.Tensor:
         for part in (layer.mixer, layer.feed_forward if self.has_ffn else None):
             if part is not None and not getattr(part, "raw_output_ok", False):
                 raise ValueError(f"{type(part).__name__} cannot give its result without the residual stream")
-        a, _ = layer.mixer_norm.forward(x32, out_t=True)
+        ahead, ctx.read_ahead = getattr(ctx, "read_ahead", None), None
+        if ahead is not None and ahead[1] == x32.data_ptr():
+            a = ahead[0]                             # the run before this one has made it with its last norm
+        else:
+            a, _ = layer.mixer_norm.forward(x32, out_t=True)
         m32 = layer.mixer.forward(a, None, ctx, cache, write)
         side = layer.side_input
         x_t = None                                  # the stream in the storage type, where a pass has made it
@@ -106,8 +121,11 @@ class Sandwich(Part):
             last = layer.ffn_out_norm
         else:
             f32, last = m32, layer.mixer_out_norm
-        if side is not None and not getattr(side, "fused", False) and _chains(last, None):
+        if side is not None and not getattr(side, "fused", False) and getattr(last, "casts_onto", False):
             x32, x_t = last.forward_onto(f32, x32, cast=True)
+        elif side is None and then is not None and type(then.arrangement) is type(self) and _chains(last, then.mixer_norm):
+            x32, made = last.forward_onto(f32, x32, then=then.mixer_norm)
+            ctx.read_ahead = (made, x32.data_ptr())
         else:
             x32 = last.forward_onto(f32, x32)
         if side is not None:
@@ -167,9 +185,8 @@ class ParallelResidual(Part):
 
 
 def _chains(norm, then) -> bool:
-    """Whether ``norm.forward_onto`` can make a second result in the same pass (``then``: another norm of its
-    kind, or None for the plain sum in the storage type)."""
-    return getattr(norm, "chains_onto", False) and (then is None or type(then) is type(norm))
+    """Whether ``norm.forward_onto(..., then=then)`` makes that norm of the sum in the same pass."""
+    return getattr(norm, "chains_onto", False) and norm.chains_with(then)
 
 
 class HyperConnections(Part):

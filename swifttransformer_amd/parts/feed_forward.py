@@ -54,8 +54,9 @@ class DenseFeedForward(Part):
             self.w2, self.b2 = fold_output_scale(self.w2, self.b2, tensors[self.name("out_scale")])
 
     accepts_norm = True     # forward(..., norm=part) normalises residual32 itself
+    raw_output_ok = True    # forward(..., residual32=None) returns the float result alone
 
-    def forward(self, x_t, residual32: torch.Tensor, ctx, norm=None) -> torch.Tensor:
+    def forward(self, x_t, residual32, ctx, norm=None) -> torch.Tensor:
         x_in = norm.as_input(residual32) if norm is not None else x_t
         h = K.gemm(x_in, self.w1, bias=self.b1, activation=self.activation)
         return K.gemm(h, self.w2, bias=self.b2, residual=residual32, out_f32=True, out_scale=self.residual_scale)

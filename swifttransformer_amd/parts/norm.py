@@ -6,7 +6,8 @@ the two sums in float and normalises in the storage type; here the whole
 computation is in float on the float residual stream, with the variance taken
 from centred values.  The parameter ``center`` = False gives the form that takes no mean
 off, y = x * rsqrt(mean(x^2) + eps) * gamma (+ beta) (reference src/csrc/kernel/rmsnorm.cu):
-the same kernels and the same fusion into a product, by a flag.
+the same kernels and the same fusion into a product, by a flag.  In that form, with a gain and no bias, it can also add
+its result to a stream on the way (``forward_onto``).
 
 ``DynamicTanh`` is a norm that takes no statistics of the row at all: y = tanh(alpha x) * w + b per
 element, alpha one learned number.  It can also add its result to a stream on the way
@@ -29,7 +30,8 @@ from .base import Part
 class LayerNorm(Part):
     """params: eps (float), affine (bool), center (bool, default True; False: root-mean-square norm),
     bias (bool, default = affine: whether the affine part has a bias), width (int, default hidden_size),
-    scalar_gain (bool, default False: the file holds one number that multiplies every coordinate)."""
+    scalar_gain (bool, default False: the file holds one number that multiplies every coordinate), gain_offset (float,
+    default 0: the gain is the file's weight plus this)."""
 
     def __init__(self, spec, hidden_size, dtype):
         super().__init__(spec, hidden_size, dtype)
@@ -39,13 +41,17 @@ class LayerNorm(Part):
         self.has_bias = bool(spec.params.get("bias", self.affine)) and self.affine
         self.width = int(self.param("width", hidden_size))
         self.scalar_gain = bool(spec.params.get("scalar_gain", False))
+        self.gain_offset = float(spec.params.get("gain_offset", 0.0))
+        # (the root-mean-square form with a gain alone is what the stream's kernel knows)
+        self.chains_onto = not self.center and self.affine and not self.has_bias
         self.gamma: Optional[torch.Tensor] = None
         self.beta: Optional[torch.Tensor] = None
 
     def tensor_specs(self) -> List[TensorSpec]:
         if not self.affine:
             return []
-        specs = [TensorSpec(self.name("weight"), () if self.scalar_gain else (self.width,), "vector", init="gain")]
+        specs = [TensorSpec(self.name("weight"), () if self.scalar_gain else (self.width,), "vector",
+                            init="normal" if self.gain_offset else "gain")]
         if self.has_bias:
             specs.append(TensorSpec(self.name("bias"), (self.width,), "vector"))
         return specs
@@ -53,6 +59,8 @@ class LayerNorm(Part):
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         if self.affine:
             self.gamma = tensors[self.name("weight")]
+            if self.gain_offset:
+                self.gamma = self.gamma + self.gain_offset
             if self.scalar_gain:       # the kernels take a gain per coordinate
                 self.gamma = self.gamma.reshape(1).expand(self.width).contiguous()
             self.beta = tensors[self.name("bias")] if self.has_bias else None
@@ -78,12 +86,27 @@ class LayerNorm(Part):
         K.layernorm(x32, self.gamma, self.beta, self.eps, rows=rows, out_t=yt, out_f32=y32, center=self.center)
         return yt, y32
 
+    def chains_with(self, then) -> bool:
+        """Whether ``forward_onto(..., then=then)`` makes that norm of the sum in the same pass."""
+        return self.chains_onto and isinstance(then, LayerNorm) and then.chains_onto and then.width == self.width
+
+    def forward_onto(self, y32: torch.Tensor, stream32: torch.Tensor, then=None):
+        """stream32 + norm(y32), float, a new tensor (the root-mean-square form with a gain alone).  ``then`` (a norm it
+        ``chains_with``): (the sum, that norm of the sum in the storage type)."""
+        if not self.chains_onto:
+            raise ValueError("only the root-mean-square form without a bias adds its result to a stream")
+        return K.rms_onto(y32, stream32, self.gamma, self.eps, None if then is None else (then.gamma, then.eps), self.dtype)
+
 
 class DynamicTanh(Part):
     """params: width (int, default hidden_size), bias (bool, default True).  names: weight, bias, alpha
     (a tensor of no dimensions)."""
 
     chains_onto = True      # forward_onto(..., then=another of this kind / cast=True) makes a second result in its pass
+    casts_onto = True
+
+    def chains_with(self, then) -> bool:
+        return type(then) is type(self)
 
     def __init__(self, spec, hidden_size, dtype):
         super().__init__(spec, hidden_size, dtype)
