@@ -209,7 +209,7 @@ def kernel_times(args) -> int:
 
 
 def side_by_side(args, shape: str, other: str = "zitupel", beside=("opt",)) -> int:
-    """Another architecture (Zitupel, Zimorax, Gisedra, Pupalix, Fiterax) beside OPT (``beside``: or other families) at the same layer sizes (width, heads, feed-forward width of OPT
+    """Another architecture (Zitupel, Zimorax, Gisedra, Pupalix, Fiterax, Fefozen) beside OPT (``beside``: or other families) at the same layer sizes (width, heads, feed-forward width of OPT
     ``shape``; the same number of layers, 8 unless ``--layers`` says otherwise; random weights):
     decode tokens/s at batch 1, 8 and 64 from 1,024-token prompts, a 2,048-token prefill, and for
     both the per-kernel times of one decode step at batch ``--batch`` and of the prefill with their
@@ -280,6 +280,8 @@ def side_by_side(args, shape: str, other: str = "zitupel", beside=("opt",)) -> i
                     return 2 * keys * info["kv_heads"] * info["head_dim"] * info["elem"]
                 if name == "sink_attention":
                     return windowed(info)[0] * info["kv_heads"] * (info["head_dim"] + info["value_dim"]) * info["elem"]
+                if name in ("latent_rows", "latent_tiles"):       # one entry a token, its own value, for all heads
+                    return keys_read * info["head_dim"] * info["elem"]
                 return None
 
             def flops(name, info):
@@ -287,6 +289,8 @@ def side_by_side(args, shape: str, other: str = "zitupel", beside=("opt",)) -> i
                     return 4.0 * (chunked(info)[1] if info.get("window", 0) < 0 else pairs) * info["heads"] * info["head_dim"]
                 if name == "sink_attention":
                     return 2.0 * windowed(info)[1] * info["heads"] * (info["head_dim"] + info["value_dim"] + info["heads"])
+                if name in ("latent_rows", "latent_tiles"):
+                    return 2.0 * pairs * info["heads"] * (info["head_dim"] + info["value_dim"])
                 return None
             return nbytes, flops
 
@@ -602,12 +606,14 @@ def main() -> int:
                              "zitupel-125m", "zitupel-1.3b", "zitupel-6.7b",
                              "zimorax-125m", "zimorax-1.3b", "zimorax-6.7b",
                              "gisedra-125m", "gisedra-1.3b", "gisedra-6.7b",
-                             "pupalix-125m", "pupalix-1.3b", "pupalix-6.7b", "fiterax-125m", "fiterax-1.3b", "fiterax-6.7b"],
+                             "pupalix-125m", "pupalix-1.3b", "pupalix-6.7b", "fiterax-125m", "fiterax-1.3b", "fiterax-6.7b",
+                             "fefozen-125m", "fefozen-1.3b", "fefozen-6.7b"],
                     help="decode-1.3b is the default line; the others are the other model shapes; zitupel-<size>, "
                          "zimorax-<size>: that architecture beside OPT at the same layer sizes; gisedra-<size>: "
                          "Gisedra beside Zitupel and Zimorax (whose kernels are its kernels' likes) and OPT; "
                          "pupalix-<size>: Pupalix beside Gisedra, Zitupel and OPT; "
-                         "fiterax-<size>: Fiterax beside Pupalix, Gisedra, Zitupel and OPT")
+                         "fiterax-<size>: Fiterax beside Pupalix, Gisedra, Zitupel and OPT; "
+                         "fefozen-<size>: Fefozen beside Gisedra, Zimorax, Zitupel and OPT")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported")
@@ -637,6 +643,8 @@ def main() -> int:
         return side_by_side(args, args.workload.split("-", 1)[1], "gisedra", beside=("zitupel", "zimorax", "opt"))
     if args.workload.startswith("pupalix-"):
         return side_by_side(args, args.workload.split("-", 1)[1], "pupalix", beside=("gisedra", "zitupel", "opt"))
+    if args.workload.startswith("fefozen-"):
+        return side_by_side(args, args.workload.split("-", 1)[1], "fefozen", beside=("gisedra", "zimorax", "zitupel", "opt"))
     if args.workload.startswith("fiterax-"):
         return side_by_side(args, args.workload.split("-", 1)[1], "fiterax", beside=("pupalix", "gisedra", "zitupel", "opt"))
     steps = min(args.steps, CONTEXT - PROMPT_LEN)

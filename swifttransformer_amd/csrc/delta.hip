@@ -175,10 +175,12 @@ __global__ __launch_bounds__(1024) void delta_step_kernel(
 
 // ---------------------------------------------------------------- rows side by side
 // qkv [rows, channels]: the filter with SiLU, q and k at unit length (q scaled); gates [rows, 2 heads]: strength | log decay.
-// A wave takes 8 consecutive rows of one unit (a q head, a k head, 256 value channels, or the gates); the filter's inputs
-// of a row's past are the rows above in its item, before those the ring.  TM: taps at most.
+// A wave takes 8 consecutive rows of one unit: as many q and k heads as have whole segments of 64 channels in four, 256 value
+// channels, or the gates; the filter's inputs of a row's past are the rows above in its item, before those the ring.  TM:
+// taps at most; SEG: segments of a head (1, 2 or 4).
 constexpr int kInputRows = 8;
-template <int TM>
+__host__ __device__ inline int delta_head_units(const DeltaShape& sh, int seg) { return (2 * sh.qk_heads + 4 / seg - 1) / (4 / seg); }
+template <int TM, int SEG>
 __global__ __launch_bounds__(256) void delta_inputs_kernel(
     float* __restrict__ qkv, float* __restrict__ gates, const float* __restrict__ proj, int64_t stride,
     const float* __restrict__ state, int64_t slot_stride, const float* __restrict__ taps_w, const float* __restrict__ a_log,
@@ -198,22 +200,37 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(
         }
         return;
     }
-    const bool is_q = unit < sh.qk_heads, unit_vector = unit < 2 * sh.qk_heads;
-    const int64_t first = unit_vector ? (int64_t)unit * sh.dk : sh.v_off() + (int64_t)(unit - 2 * sh.qk_heads) * 256;
-    const int n = unit_vector ? sh.dk : (int)(C - first < 256 ? C - first : 256);
-    const int taps = sh.taps;
-    constexpr int L = 4;                             // channels a lane
+    const int head_units = delta_head_units(sh, SEG), taps = sh.taps;
+    const bool unit_vector = unit < head_units;
+    constexpr int L = 4;                             // channels a lane: segment e of 64
+    int64_t ch[L];
+    bool ok[L];
+    float factor[L];
+#pragma unroll
+    for (int e = 0; e < L; ++e) {
+        if (unit_vector) {
+            const int head = unit * (L / SEG) + e / SEG, c = (e % SEG) * 64 + lane;
+            ok[e] = head < 2 * sh.qk_heads && c < sh.dk;
+            ch[e] = ok[e] ? (int64_t)head * sh.dk + c : 0;
+            factor[e] = head < sh.qk_heads ? q_scale : 1.f;
+        } else {
+            const int64_t c = sh.v_off() + (int64_t)(unit - head_units) * 256 + 64 * e + lane;
+            ok[e] = c < C;
+            ch[e] = ok[e] ? c : 0;
+            factor[e] = 1.f;
+        }
+    }
     float x[kInputRows + TM - 1][L], w[TM][L];
 #pragma unroll
     for (int i = 0; i < kInputRows + TM - 1; ++i) {
         const int t = min(max(t0 + i - (TM - 1), 0), num_tokens - 1);
 #pragma unroll
-        for (int e = 0; e < L; ++e) x[i][e] = proj[(int64_t)t * stride + first + min(lane + 64 * e, n - 1)];
+        for (int e = 0; e < L; ++e) x[i][e] = proj[(int64_t)t * stride + ch[e]];
     }
 #pragma unroll
     for (int j = 0; j < TM; ++j)
 #pragma unroll
-        for (int e = 0; e < L; ++e) w[j][e] = j < taps ? taps_w[(int64_t)(taps - 1 - j) * C + first + min(lane + 64 * e, n - 1)] : 0.f;
+        for (int e = 0; e < L; ++e) w[j][e] = j < taps ? taps_w[(int64_t)(taps - 1 - j) * C + ch[e]] : 0.f;
 #pragma unroll
     for (int r = 0; r < kInputRows; ++r) {
         const int t = t0 + r;
@@ -234,20 +251,25 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(
             } else if (pos >= j) {
 #pragma unroll
                 for (int e = 0; e < L; ++e)
-                    acc[e] = fmaf(w[j][e], ring[(int64_t)((pos - j) % taps) * C + first + min(lane + 64 * e, n - 1)], acc[e]);
+                    acc[e] = fmaf(w[j][e], ring[(int64_t)((pos - j) % taps) * C + ch[e]], acc[e]);
             }
         }
-        float ss = 0.f;
 #pragma unroll
-        for (int e = 0; e < L; ++e) {
-            acc[e] = lane + 64 * e < n ? delta_silu(acc[e]) : 0.f;
-            ss = fmaf(acc[e], acc[e], ss);
+        for (int e = 0; e < L; ++e) acc[e] = ok[e] ? delta_silu(acc[e]) : 0.f;
+        if (unit_vector) {
+#pragma unroll
+            for (int h = 0; h < L / SEG; ++h) {
+                float ss = 0.f;
+#pragma unroll
+                for (int e = h * SEG; e < (h + 1) * SEG; ++e) ss = fmaf(acc[e], acc[e], ss);
+                const float f = 1.f / sqrtf(wave_sum(ss) + unit_eps);
+#pragma unroll
+                for (int e = h * SEG; e < (h + 1) * SEG; ++e) acc[e] *= f * factor[e];
+            }
         }
-        float f = 1.f;
-        if (unit_vector) f = (is_q ? q_scale : 1.f) / sqrtf(wave_sum(ss) + unit_eps);
 #pragma unroll
         for (int e = 0; e < L; ++e)
-            if (lane + 64 * e < n) qkv[(int64_t)t * C + first + lane + 64 * e] = acc[e] * f;
+            if (ok[e]) qkv[(int64_t)t * C + ch[e]] = acc[e];
     }
 }
 
@@ -353,8 +375,9 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
 // Grid (heads, blocks of 16 value channels, items): walks a request's chunks.  wv becomes U, start [chunk, head, dk, dv]
 // receives the chunks' start states.  A wave owns 16 rows of U and every fourth tile of 16 key channels of S; both meet in
 // LDS: S [16 KT][20] | U [64][20].  The matrix instruction's four depth slots are key channels (rows) 4 g + r, so that the
-// results of one product are the operands of the next as they lie.  KT: dk <= 16 KT.
-template <int KT>
+// results of one product are the operands of the next as they lie.  KT: dk <= 16 KT; AHEAD: chunks whose operands are on
+// their way at a time (a trip to memory takes longer than a chunk).
+template <int KT, int AHEAD>
 __global__ __launch_bounds__(256) void delta_carry_kernel(
     float* __restrict__ wv, const float* __restrict__ wk, const float* __restrict__ kt, const float* __restrict__ fall,
     float* __restrict__ start, float* __restrict__ state, int64_t slot_stride, const int* __restrict__ item_len,
@@ -384,9 +407,10 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(
             if (wave + 4 * m < KT) ss[kk][r16] = S[m][r];
         }
     const bool quads = dk % 4 == 0;
-    floatx4 fk[KT], ft[MT][4], fv;
-    float fg;
-    auto load = [&](int c) {
+    struct Operands {
+        floatx4 fk[KT], ft[MT][4], fv;
+    };
+    auto load = [&](Operands& p, int c) {
         const int64_t at = (int64_t)(first + c) * sh.heads + head;
         const float* a = wk + (at * kChunkRows + 16 * wave + r16) * dk;
 #pragma unroll
@@ -394,10 +418,10 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(
             const int kk = 16 * t + 4 * g;
             if (quads) {
                 const float4 v = *reinterpret_cast<const float4*>(a + min(kk, dk - 4));
-                fk[t] = kk < dk ? floatx4{v.x, v.y, v.z, v.w} : floatx4{0.f, 0.f, 0.f, 0.f};
+                p.fk[t] = kk < dk ? floatx4{v.x, v.y, v.z, v.w} : floatx4{0.f, 0.f, 0.f, 0.f};
             } else {
 #pragma unroll
-                for (int r = 0; r < 4; ++r) { const float v = a[min(kk + r, dk - 1)]; fk[t][r] = kk + r < dk ? v : 0.f; }
+                for (int r = 0; r < 4; ++r) { const float v = a[min(kk + r, dk - 1)]; p.fk[t][r] = kk + r < dk ? v : 0.f; }
             }
         }
 #pragma unroll
@@ -407,30 +431,25 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(
 #pragma unroll
             for (int s = 0; s < 4; ++s) {
                 const float4 v = *reinterpret_cast<const float4*>(b + 16 * s + 4 * g);
-                ft[m][s] = floatx4{v.x, v.y, v.z, v.w};       // (rows of channels past dk give rows of S that are not kept)
+                p.ft[m][s] = floatx4{v.x, v.y, v.z, v.w};     // (rows of channels past dk give rows of S that are not kept)
             }
         }
 #pragma unroll
-        for (int r = 0; r < 4; ++r) fv[r] = wv[(at * kChunkRows + 16 * wave + 4 * g + r) * dv + colc];
-        fg = fall[at];
+        for (int r = 0; r < 4; ++r) p.fv[r] = wv[(at * kChunkRows + 16 * wave + 4 * g + r) * dv + colc];
     };
-    load(0);
-    __syncthreads();
-    for (int c = 0; c < chunks; ++c) {
+    // (a lane holds the factor of chunk lane of the present 64: a load that is the same for all lanes would be a scalar one,
+    // and every barrier waits for those)
+    float falls = 0.f;
+    auto step = [&](Operands& p, int c) {
+        if ((c & 63) == 0) falls = fall[(int64_t)(first + min(c + lane, chunks - 1)) * sh.heads + head];
+        const float keep = __shfl(falls, c & 63, 64);
         const int64_t at = (int64_t)(first + c) * sh.heads + head;
         floatx4 acc = floatx4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int t = 0; t < KT; ++t)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(fk[t][r], ss[16 * t + 4 * g + r][r16], acc, 0, 0, 0);
-        floatx4 kts[MT][4];
-#pragma unroll
-        for (int m = 0; m < MT; ++m)
-#pragma unroll
-            for (int s = 0; s < 4; ++s) kts[m][s] = ft[m][s];
-        const floatx4 u = fv - acc;
-        const float keep = fg;
-        if (c + 1 < chunks) load(c + 1);             // on their way during the second product
+            for (int r = 0; r < 4; ++r) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(p.fk[t][r], ss[16 * t + 4 * g + r][r16], acc, 0, 0, 0);
+        const floatx4 u = p.fv - acc;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             su[16 * wave + 4 * g + r][r16] = u[r];
@@ -451,7 +470,7 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(
 #pragma unroll
             for (int s = 0; s < 4; ++s)
 #pragma unroll
-                for (int r = 0; r < 4; ++r) d = __builtin_amdgcn_mfma_f32_16x16x4f32(kts[m][s][r], su[16 * s + 4 * g + r][r16], d, 0, 0, 0);
+                for (int r = 0; r < 4; ++r) d = __builtin_amdgcn_mfma_f32_16x16x4f32(p.ft[m][s][r], su[16 * s + 4 * g + r][r16], d, 0, 0, 0);
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int kk = 16 * (wave + 4 * m) + 4 * g + r;
@@ -459,7 +478,17 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(
                 ss[kk][r16] = S[m][r];
             }
         }
+        if (c + AHEAD < chunks) load(p, c + AHEAD);
         __syncthreads();
+    };
+    Operands ops[AHEAD];
+#pragma unroll
+    for (int b = 0; b < AHEAD; ++b) load(ops[b], min(b, chunks - 1));
+    __syncthreads();
+    for (int c0 = 0; c0 < chunks; c0 += AHEAD) {
+#pragma unroll
+        for (int b = 0; b < AHEAD; ++b)
+            if (c0 + b < chunks) step(ops[b], c0 + b);       // uniform
     }
 #pragma unroll
     for (int m = 0; m < MT; ++m)
@@ -693,12 +722,15 @@ extern "C" int st_delta_chunks(void* out, const float* proj, int64_t stride, flo
     const int64_t chunks = num_rows / kChunkRows + num_items;  // every item's last chunk may be a short one
     ST_CHECK(scratch_chunks >= chunks, "delta_chunks: scratch for %lld chunks, %lld needed", (long long)scratch_chunks, (long long)chunks);
     ST_CHECK(chunks <= 65535 && num_items <= 65535, "delta_chunks: too many chunks or items");
-    const int units = 2 * qk_heads + (heads * value_dim + 255) / 256 + 1;
+    const int seg = key_dim <= 64 ? 1 : key_dim <= 128 ? 2 : 4;
+    const int units = delta_head_units(sh, seg) + (heads * value_dim + 255) / 256 + 1;
     const dim3 grid_in((num_rows + kInputRows - 1) / kInputRows, (units + 3) / 4);
-#define ST_DI(TM)                                                                                                      \
-    delta_inputs_kernel<TM><<<grid_in, 256, 0, stream>>>(qkv, gates, proj, stride, state, slot_stride, taps_w, a_log, dt_bias, \
+#define ST_DI(TM, SEG)                                                                                                 \
+    delta_inputs_kernel<TM, SEG><<<grid_in, 256, 0, stream>>>(qkv, gates, proj, stride, state, slot_stride, taps_w, a_log, dt_bias, \
         token_item, positions, item_tok_off, item_slot, num_rows, units, sh, q_scale, unit_eps)
-    if (taps <= 4) ST_DI(4); else ST_DI(8);
+#define ST_DI_S(TM) do { if (seg == 1) ST_DI(TM, 1); else if (seg == 2) ST_DI(TM, 2); else ST_DI(TM, 4); } while (0)
+    if (taps <= 4) ST_DI_S(4); else ST_DI_S(8);
+#undef ST_DI_S
 #undef ST_DI
     ST_LAUNCH_CHECK("delta_chunks (inputs)");
     // 16-byte loads where every section of a row and every row of the scratch starts on a 16-byte border
@@ -723,12 +755,12 @@ extern "C" int st_delta_chunks(void* out, const float* proj, int64_t stride, flo
 #undef ST_DP2
     ST_LAUNCH_CHECK("delta_chunks (prep)");
     const dim3 grid_c(heads, (value_dim + 15) / 16, num_items);
-#define ST_DC(KT) delta_carry_kernel<KT><<<grid_c, 256, 0, stream>>>(wv, wk, kt, fall, start, state, slot_stride, item_len, item_slot, sh)
-    if (key_dim <= 16) ST_DC(1);
-    else if (key_dim <= 32) ST_DC(2);
-    else if (key_dim <= 64) ST_DC(4);
-    else if (key_dim <= 128) ST_DC(8);
-    else ST_DC(16);
+#define ST_DC(KT, AHEAD) delta_carry_kernel<KT, AHEAD><<<grid_c, 256, 0, stream>>>(wv, wk, kt, fall, start, state, slot_stride, item_len, item_slot, sh)
+    if (key_dim <= 16) ST_DC(1, 4);
+    else if (key_dim <= 32) ST_DC(2, 4);
+    else if (key_dim <= 64) ST_DC(4, 4);
+    else if (key_dim <= 128) ST_DC(8, 2);
+    else ST_DC(16, 1);
 #undef ST_DC
     ST_LAUNCH_CHECK("delta_chunks (carry)");
 #define ST_DO_E(T, KQ, NV, VEC)                                                                                        \

@@ -134,9 +134,12 @@ extern "C" int st_latent_inputs(void* cq, int cq_width, const float* gain_q, int
         tail_off, tail, freq, half, tail_mult, entry, x, x_stride, token_item, positions, block_table, max_pages, page_size,    \
         num_tokens, eps)
     const int most = cache && rank > q_rank ? rank : q_rank;
-    if (dtype == kF32) { if (most <= 256) ST_LI(float, 4); else ST_LI(float, 24); }
-    else if (dtype == kBF16) { if (most <= 256) ST_LI(bf16_t, 4); else ST_LI(bf16_t, 24); }
+#define ST_LI_T(T) do { if (most <= 128) ST_LI(T, 2); else if (most <= 256) ST_LI(T, 4); else if (most <= 512) ST_LI(T, 8); \
+                        else if (most <= 1024) ST_LI(T, 16); else ST_LI(T, 24); } while (0)
+    if (dtype == kF32) ST_LI_T(float);
+    else if (dtype == kBF16) ST_LI_T(bf16_t);
     else ST_CHECK(false, "latent_inputs: unknown dtype %d", dtype);
+#undef ST_LI_T
 #undef ST_LI
     ST_LAUNCH_CHECK("latent_inputs");
     return 0;

@@ -428,7 +428,8 @@ def test_peaked_attention_far_back_and_at_page_borders(models, tmp_path, dtype, 
     parts say which key each query of the last layer weighs most: some far back, some at page borders, some the
     sequence's first."""
     _, cfg0, w0 = models[name]
-    boost = 30.0 if dtype == "float32" else 3.0
+    # (behind a peaked layer the next one's scores carry its rounding on)
+    boost = (30.0 if len(picked) == 1 else 10.0) if dtype == "float32" else 3.0
 
     def change(m, w, p):
         m["scale"] = m["scale"] * boost
@@ -489,14 +490,13 @@ def test_a_state_that_keeps_a_token_for_long(models, tmp_path, dtype):
         w[p + "mix.A_log"] = torch.full_like(w[p + "mix.A_log"], -8.0)
         w[p + "mix.b"] *= 0.3
     folder, cfg, w = _layers_alone(cfg0, w0, [0], tmp_path, change)
-    cfg["vocab"]
     seqs = {0: tiny.prompt(300, cfg["vocab"], 5), 1: tiny.prompt(120, cfg["vocab"], 6)}
     seqs[0][0] = 60                                             # a token of its own at the start, asked for again at the end
     seqs[0][1:299] = [t % 60 for t in seqs[0][1:299]]
     seqs[0][299] = 60
     refs = {r: plain.logits(cfg, w, s).numpy() for r, s in seqs.items()}
     other = plain.logits(cfg, w, [0] + seqs[0][1:]).numpy()
-    assert np.abs(other[299] - refs[0][299]).max() > 0.1 * refs[0][299].std()       # the first token shows at the end
+    assert np.abs(other[299] - refs[0][299]).max() > 0.05 * refs[0][299].std()      # the first token shows at the end
     runner = make_runner(folder, dtype, 16, 40, record_after=2, max_seqs=2)
     run_schedule(runner, seqs, refs, [[(0, 40), (1, 2)]] + [[(0, 1), (1, 1)]] * 30 + [[(1, 70), (0, 1)], [(0, 2), (1, 18)], [(0, 150)]] +
                  [[(0, 1)]] * 77, dtype, "beside another", loosen=3.0)
