@@ -7,7 +7,7 @@
 //
 // With one key head the queries of all heads of a token read the same keys, so rows of the products are (token, head)
 // pairs, flattened in memory order:
-//   tiles   64 tokens of one item are 64 * heads rows, cut into workgroups of 64 or 128 rows (prompts and portions);
+//   tiles   64 tokens of one item are 64 * heads rows, cut into workgroups of 64 rows (prompts and portions);
 //   rows    the heads of one token, keys split over workgroups and over the waves of one (decoded tokens): every entry is
 //           read once for all heads; partial results (normalised, with their log-sum-exps) are merged by the reader.
 // A block of entries lies in LDS once and serves both products: S^T = K Q^T reads its rows, O^T += V^T P^T reads it
@@ -113,6 +113,25 @@ template <int CH> __device__ inline int latent_swizzle(int row) {
     return (((row >> 2) & 1) << 1) | ((row >> 3) & 1);
 }
 
+// cosine and sine (times rot_mult) of the turning pairs at the positions of a workgroup's tokens: [tokens][rot_half] in LDS.
+// (Once a position in LDS instead of once a lane: the accurate functions, inlined at every place of a query that may
+// turn, were four fifths of the kernel's code, and a short launch is as long as its code takes to arrive.)
+template <int THREADS>
+__device__ inline void latent_turns(const LatentArgs& a, const LatentRows& r, int rows, float2* turns) {
+    const int last = min(rows, r.total - r.fr0) - 1, first = r.fr0 / a.heads, tokens = (r.fr0 + last) / a.heads - first + 1;
+#pragma unroll 1
+    for (int i = threadIdx.x; i < tokens * a.rot_half; i += THREADS) {
+        const int t = i / a.rot_half;
+        const float ang = (float)(r.pos0 + first + t) * a.freq[i - t * a.rot_half];
+        turns[i] = make_float2(cosf(ang) * a.rot_mult, sinf(ang) * a.rot_mult);
+    }
+}
+// tokens of a workgroup at most
+__host__ __device__ inline int latent_tokens(int rows, int heads) {
+    const int n = (rows - 1 + heads - 1) / heads + 1;
+    return n < kTileTokens ? n : kTileTokens;
+}
+
 __device__ inline float lo_half(uint32_t w) { return __uint_as_float(w << 16); }
 __device__ inline float hi_half(uint32_t w) { return __uint_as_float(w & 0xffff0000u); }
 
@@ -125,7 +144,8 @@ __global__ __launch_bounds__(64 * RW * KW) void latent_attn_kernel(const LatentA
     static_assert(NI * 64 * RW == DK * CH && NKT % 2 == 0, "whole loads");
     extern __shared__ uint4 dyn[];
     char* lds_all = reinterpret_cast<char*>(dyn);    // a group of waves: [2 buffers][DK rows][ROWB]
-    int* s_bt = reinterpret_cast<int*>(lds_all + KW * 2 * BUF);
+    float2* turns = reinterpret_cast<float2*>(lds_all + KW * 2 * BUF);
+    int* s_bt = reinterpret_cast<int*>(turns + (a.rot_half ? (TILES ? latent_tokens(ROWS, a.heads) : 1) * a.rot_half + 4 : 0));
     LatentRows rows;
     if (!latent_find_rows<TILES>(a, ROWS, rows)) return;
     const LatentKeys keys = latent_keys<TILES>(a, rows, ROWS, DK);
@@ -143,6 +163,7 @@ __global__ __launch_bounds__(64 * RW * KW) void latent_attn_kernel(const LatentA
         for (int i = tid; i < p_n; i += 64 * RW * KW) s_bt[i] = bt[i];
     }
     // ---- queries: lane (row r16 of a subtile, group g) holds dims 32 s + 8 g .. + 7, turned where they meet the turned part
+    uint4 qraw[QT][HDP];
     bf16x8 qf[QT][HDP];
     int qpos[QT], qhead[QT];
     bool qvalid[QT];
@@ -157,17 +178,30 @@ __global__ __launch_bounds__(64 * RW * KW) void latent_attn_kernel(const LatentA
 #pragma unroll
         for (int s = 0; s < HDP; ++s) {
             const int d = 32 * s + 8 * g;
-            uint4 v = make_uint4(0, 0, 0, 0);
-            if (qvalid[t] && d < a.entry) v = *reinterpret_cast<const uint4*>(qrow + d);
+            const uint4 v = *reinterpret_cast<const uint4*>(qrow + min(d, a.entry - 8));
+            qraw[t][s] = qvalid[t] && d < a.entry ? v : make_uint4(0, 0, 0, 0);
+        }
+    }
+    if (a.rot_half) {
+        latent_turns<64 * RW * KW>(a, rows, ROWS, turns);
+        __syncthreads();
+    }
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+        const float2* mine = turns + (qpos[t] - rows.pos0 - rows.fr0 / a.heads) * a.rot_half;
+#pragma unroll
+        for (int s = 0; s < HDP; ++s) {
+            const int d = 32 * s + 8 * g;
+            uint4 v = qraw[t][s];
             const int pair0 = (d - a.rot_off) >> 1;
             if (d >= a.rot_off && pair0 < a.rot_half) {
                 uint32_t w[4] = {v.x, v.y, v.z, v.w};
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
-                    if (pair0 + e >= a.rot_half) continue;
-                    const float ang = (float)qpos[t] * a.freq[pair0 + e];
-                    const float c = cosf(ang) * a.rot_mult, sn = sinf(ang) * a.rot_mult, u = lo_half(w[e]), x = hi_half(w[e]);
-                    w[e] = pack_bf16x2(u * c - x * sn, x * c + u * sn);
+                    const float2 cs = mine[pair0 + e];           // (past the last pair: whatever follows, not used)
+                    const float u = lo_half(w[e]), x = hi_half(w[e]);
+                    const uint32_t turned = pack_bf16x2(u * cs.x - x * cs.y, x * cs.x + u * cs.y);
+                    w[e] = pair0 + e < a.rot_half ? turned : w[e];
                 }
                 v = make_uint4(w[0], w[1], w[2], w[3]);
             }
@@ -199,7 +233,11 @@ __global__ __launch_bounds__(64 * RW * KW) void latent_attn_kernel(const LatentA
     // ---- readers' offsets.  As keys: row r16 of a subtile, chunk 4 s + g.  Transposed: a lane of 16 reads 4 dims (8 bytes)
     // of row 4 g + r16 / 4, chunk 2 dt + (r16 % 4) / 2, and receives dim r16 of four rows
     const int sw_k = latent_swizzle<CH>(r16), vrow = 4 * g + (r16 >> 2), sw_v = latent_swizzle<CH>(vrow);
-    const int kbase = r16 * ROWB, vbase = vrow * ROWB + ((r16 & 1) << 3), vsub = (r16 & 3) >> 1;
+    int koff[HDP], voff[DT];
+#pragma unroll
+    for (int s = 0; s < HDP; ++s) koff[s] = r16 * ROWB + (((4 * s + g) ^ sw_k) << 4);
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) voff[dt] = vrow * ROWB + (((2 * dt + ((r16 & 3) >> 1)) ^ sw_v) << 4) + ((r16 & 1) << 3);
 
     // running maximum (log2 units, from a finite floor), accumulators, and the normaliser as one more row of the product
     float ms[QT];
@@ -239,7 +277,7 @@ __global__ __launch_bounds__(64 * RW * KW) void latent_attn_kernel(const LatentA
 #pragma unroll
             for (int kt = 0; kt < NKT; ++kt)
                 k8[kt] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(
-                    ks + kt * 16 * ROWB + kbase + (((4 * s + g) ^ sw_k) << 4)));
+                    ks + kt * 16 * ROWB + koff[s]));
 #pragma unroll
             for (int t = 0; t < QT; ++t)
 #pragma unroll
@@ -295,7 +333,7 @@ __global__ __launch_bounds__(64 * RW * KW) void latent_attn_kernel(const LatentA
 #pragma unroll
             for (int dt = 0; dt < DT; ++dt) {
                 if (16 * dt >= a.out_dim) continue;  // uniform
-                const char* at = ks + 32 * u * ROWB + vbase + (((2 * dt + vsub) ^ sw_v) << 4);
+                const char* at = ks + 32 * u * ROWB + voff[dt];
                 const short4v lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(ST_LDS_PTR(short4v, at));
                 const short4v hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(ST_LDS_PTR(short4v, at + 16 * ROWB));
                 const uint2 lo2 = __builtin_bit_cast(uint2, lo), hi2 = __builtin_bit_cast(uint2, hi);
@@ -396,7 +434,8 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(const LatentArgs a
     constexpr int DK = kLatentF32Keys, KS = 16 * ET + 4, ROWS = 64;
     extern __shared__ uint4 dyn[];
     float* ks = reinterpret_cast<float*>(dyn);       // [DK][KS]
-    int* s_bt = reinterpret_cast<int*>(ks + DK * KS);
+    float2* turns = reinterpret_cast<float2*>(ks + DK * KS);
+    int* s_bt = reinterpret_cast<int*>(turns + (a.rot_half ? (TILES ? latent_tokens(ROWS, a.heads) : 1) * a.rot_half + 4 : 0));
     LatentRows rows;
     if (!latent_find_rows<TILES>(a, ROWS, rows)) return;
     const LatentKeys keys = latent_keys<TILES>(a, rows, ROWS, DK);
@@ -412,7 +451,12 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(const LatentArgs a
     const bool qvalid = i < rows.total;
     const int ii = qvalid ? i : rows.fr0, token = ii / a.heads, qhead = ii - token * a.heads, qpos = rows.pos0 + token;
     floatx4 qf[ET];                                  // dims 16 j + 4 g .. + 3
+    if (a.rot_half) {
+        latent_turns<256>(a, rows, ROWS, turns);
+        __syncthreads();
+    }
     {
+        const float2* mine = turns + (token - rows.fr0 / a.heads) * a.rot_half;
         const float* qrow = reinterpret_cast<const float*>(a.q) + (rows.token0 + token) * a.q_stride + (int64_t)qhead * a.entry;
 #pragma unroll
         for (int j = 0; j < ET; ++j) {
@@ -424,10 +468,10 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(const LatentArgs a
 #pragma unroll
                 for (int e = 0; e < 2; ++e) {
                     if (pair0 + e >= a.rot_half) continue;
-                    const float ang = (float)qpos * a.freq[pair0 + e];
-                    const float c = cosf(ang) * a.rot_mult, sn = sinf(ang) * a.rot_mult, u = v[2 * e], x = v[2 * e + 1];
-                    v[2 * e] = u * c - x * sn;
-                    v[2 * e + 1] = x * c + u * sn;
+                    const float2 cs = mine[pair0 + e];
+                    const float u = v[2 * e], x = v[2 * e + 1];
+                    v[2 * e] = u * cs.x - x * cs.y;
+                    v[2 * e + 1] = x * cs.x + u * cs.y;
                 }
             }
             qf[j] = v;
@@ -671,15 +715,19 @@ static int64_t latent_table(const LatentArgs& a, bool tiles, int block) {
     return pages < a.max_pages ? pages : a.max_pages;
 }
 
+static size_t latent_turn_bytes(const LatentArgs& a, bool tiles, int rows) {
+    return a.rot_half ? ((size_t)(tiles ? latent_tokens(rows, a.heads) : 1) * a.rot_half + 4) * sizeof(float2) : 0;
+}
+
 template <bool TILES, int HDP, int QT, int NKT, int RW, int KW>
 static int launch_latent(const LatentArgs& a, int list, hipStream_t stream) {
     auto kernel = latent_attn_kernel<TILES, HDP, QT, NKT, RW, KW>;
     constexpr size_t bufs = (size_t)KW * 2 * 16 * NKT * HDP * 64;
     constexpr size_t merge = (size_t)(KW - 1) * RW * 64 * QT * (2 + 8 * HDP) * sizeof(float);
-    const size_t table = (size_t)latent_table(a, TILES, 16 * NKT) * sizeof(int);
+    constexpr int rows = RW * QT * 16;
+    const size_t table = (size_t)latent_table(a, TILES, 16 * NKT) * sizeof(int) + latent_turn_bytes(a, TILES, rows);
     const size_t lds = bufs + table > merge ? bufs + table : merge;
     if (latent_raise_lds(reinterpret_cast<const void*>(kernel), lds)) return 1;
-    constexpr int rows = RW * QT * 16;
     const int x = ((TILES ? kTileTokens : 1) * a.heads + rows - 1) / rows;
     LatentArgs args = a;
     if (TILES) {
@@ -695,7 +743,8 @@ static int launch_latent(const LatentArgs& a, int list, hipStream_t stream) {
 template <bool TILES, int ET>
 static int launch_latent_f32(const LatentArgs& a, int list, hipStream_t stream) {
     auto kernel = latent_attn_f32_kernel<TILES, ET>;
-    const size_t lds = sizeof(float) * ((size_t)kLatentF32Keys * (16 * ET + 4)) + (size_t)latent_table(a, TILES, kLatentF32Keys) * sizeof(int);
+    const size_t lds = sizeof(float) * ((size_t)kLatentF32Keys * (16 * ET + 4)) + (size_t)latent_table(a, TILES, kLatentF32Keys) * sizeof(int) +
+                       latent_turn_bytes(a, TILES, 64);
     if (latent_raise_lds(reinterpret_cast<const void*>(kernel), lds)) return 1;
     const int x = ((TILES ? kTileTokens : 1) * a.heads + 63) / 64;
     LatentArgs args = a;
@@ -720,12 +769,12 @@ static int latent_dispatch(const LatentArgs& a, int list, int dtype, hipStream_t
     }
     // (an entry runs in the next larger instance, its missing chunks zeros in LDS)
     const int hdp = (a.entry + 31) / 32;
-    // tiles: four waves of 32 rows (16 where entries are large), blocks of 64 keys (32); rows: one wave of 16 or 32 rows,
+    // tiles: four waves of 16 rows, blocks of 64 keys (32 where entries are large); rows: one or two waves of 16 rows,
     // four (two) shares of the keys, blocks of 32 keys
 #define ST_LT(H)                                                                                                       \
     if (hdp <= H) {                                                                                                    \
-        if constexpr (TILES) return launch_latent<TILES, H, 2, 4, 4, 1>(a, list, stream);                              \
-        else return a.heads <= 16 ? launch_latent<TILES, H, 1, 2, 1, 4>(a, list, stream) : launch_latent<TILES, H, 2, 2, 1, 4>(a, list, stream); \
+        if constexpr (TILES) return launch_latent<TILES, H, 1, 4, 4, 1>(a, list, stream);                              \
+        else return a.heads <= 16 ? launch_latent<TILES, H, 1, 2, 1, 4>(a, list, stream) : launch_latent<TILES, H, 1, 2, 2, 4>(a, list, stream); \
     }
 #define ST_LB(H)                                                                                                       \
     if (hdp <= H) {                                                                                                    \
