@@ -170,8 +170,8 @@ def test_a_longer_sequence_leaves_earlier_logits_and_every_mechanism_moves_them(
             t[:, :-1] = 0.0                                      # (the taps before the row's own)
             assert w[key].shape[1] == 1 or moves({key: t}) > 1e-3, key
         elif ".e" not in key:
-            # (a constant on every router logit changes nothing)
-            assert moves({key: 1.5 * t if key.endswith("router") else t + 0.5}) > 1e-3, key
+            # (a constant on every router logit changes nothing, and one expert's weight alone goes in the norm behind)
+            assert moves({key: torch.roll(t, 1, 0) if key.endswith("router") else t + 0.5}) > 1e-3, key
 
 
 @pytest.mark.parametrize("name", [n for n in tiny.CONFIGS if tiny.reserved(tiny.CONFIGS[n])])
