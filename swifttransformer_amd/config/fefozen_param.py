@@ -70,9 +70,9 @@ class FefozenHyperParam:
         heads = _need(m, "heads", w, (int,), 1)
         if heads % _need(m, "kv_heads", w, (int,), 1):
             raise ConfigError(f"config.json: {w}.heads must be a multiple of kv_heads")
-        for key in ("dim", "vdim"):
-            if _need(m, key, w, (int,), 1) > 256:
-                raise ConfigError(f"config.json: {w}.{key}: up to 256 channels a head, got {m[key]}")
+        if _need(m, "dim", w, (int,), 1) > 256:
+            raise ConfigError(f"config.json: {w}.dim: up to 256 key channels a head, got {m['dim']}")
+        _need(m, "vdim", w, (int,), 1)
         if _need(m, "conv", w, (int,), 1) > 8:
             raise ConfigError(f"config.json: {w}.conv: 1 to 8 taps, got {m['conv']}")
 

@@ -18,7 +18,7 @@ def _norm(hp: FefozenHyperParam, name: str) -> PartSpec:
 
 def _mixer(hp: FefozenHyperParam, kind: str, p: str, mx: dict) -> PartSpec:
     if kind == "delta":
-        return PartSpec("delta_rule",
+        return PartSpec("gated_delta",
                         {"num_heads": mx["heads"], "num_qk_heads": mx["kv_heads"], "key_dim": mx["dim"], "value_dim": mx["vdim"],
                          "taps": mx["conv"], "eps": hp.norm_eps, "unit_eps": 1e-6},
                         {"q": f"{p}.q", "k": f"{p}.k", "v": f"{p}.v", "gate": f"{p}.g", "q_conv": f"{p}.q.conv",

@@ -45,7 +45,6 @@ register_part("mixer", "parallel", ParallelMixers)
 register_part("side_input", "token_side", TokenSideInput)
 from .arrangement import HyperConnections, ParallelResidual
 from .embedding import HashedPairEmbedding
-from .delta import FusedDeltaRule
 from .feed_forward import GatedFeedForward
 from .gated_latent import GatedLatentAttention
 from .matrix_memory import MatrixMemory
@@ -62,4 +61,3 @@ register_part("mixer", "matrix_memory", MatrixMemory)
 register_part("mixer", "unit_qk_attention", UnitQueryKeyAttention)
 register_part("norm", "group_rms", GroupRmsNorm)
 register_part("mixer", "gated_latent_attention", GatedLatentAttention)
-register_part("mixer", "delta_rule", FusedDeltaRule)

@@ -12,14 +12,19 @@
     S <- a S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
     out = Wo (unit(o) * g * silu(Wg h))
 
+The delta rule has two routes.  Heads of up to 256 value channels: one product makes q, k, v, the gate and the logits of beta and
+a as floats, a step of single tokens then is one kernel (filter, unit vectors, gates, state, read-out, norm and gate), and
+other steps go by chunks of rows with float products on the matrix cores and a carry of the state between chunks
+(``K.delta_rule``).  Wider heads: a kernel a mechanism around the scan that walks token by token (``K.state_scan``).
+
 Per request both keep the recurrent state (float) and the convolution's last ``taps - 1`` inputs in one
-flat float state (``CacheNeed("state")``), carried from step to step, so prompts, portions and single
+flat float state (``CacheNeed("state")``; the first route of the delta rule keeps the inputs as a ring of ``taps``), carried from step to step, so prompts, portions and single
 tokens run through the same kernels.  Products take the engine's storage type; step sizes, decays,
 gates of the recurrence, unit norms, the state and the sums over it are float.  A per-feature factor on
 the result (``out_scale``) is folded into Wo.  The reference has no such mixers."""
 from __future__ import annotations
 
-from typing import Dict, List
+from typing import Dict, List, Optional
 
 import torch
 
@@ -118,8 +123,11 @@ class Mamba2Mixer(_RecurrentMixer):
 
 
 class GatedDeltaRule(_RecurrentMixer):
-    """params: num_heads, num_qk_heads, key_dim, value_dim, taps, eps (of the output's unit norm), unit_eps
-    (of the unit vectors, default 1e-6), out_scale (bool)."""
+    """params: num_heads, num_qk_heads (default num_heads: heads share q and k in groups of neighbours), key_dim (up to 256),
+    value_dim, taps (1 to 8), eps (of the output's unit norm), unit_eps (of the unit vectors, default 1e-6), out_scale (bool).
+    names: q, k, v, gate, q_conv, k_conv, v_conv [channels, taps], write, decay, a_log, dt_bias, norm [value_dim], out."""
+
+    raw_output_ok = True     # forward(..., residual32=None) returns the mixer's result alone
 
     def __init__(self, spec, hidden_size, dtype):
         super().__init__(spec, hidden_size, dtype)
@@ -134,12 +142,19 @@ class GatedDeltaRule(_RecurrentMixer):
         if self.num_heads % self.num_qk_heads:
             raise ValueError(f"{self.num_heads} heads do not divide over {self.num_qk_heads} query/key heads")
         if self.key_dim > 256 or not 1 <= self.taps <= 8:
-            raise ValueError(f"the scan takes up to 256 key channels (got {self.key_dim}), the filter 1 to 8 taps "
+            raise ValueError(f"the delta rule takes up to 256 key channels (got {self.key_dim}), the filter 1 to 8 taps "
                              f"(got {self.taps})")
         self.qk_size = self.num_qk_heads * self.key_dim
         self.v_size = self.num_heads * self.value_dim
         self.conv_channels = 2 * self.qk_size + self.v_size
         self.state_dims = (self.num_heads, self.key_dim, self.value_dim)
+        self.sizes = (self.num_heads, self.num_qk_heads, self.key_dim, self.value_dim)
+        self.fused = self.value_dim <= 256
+
+    def cache_need(self) -> CacheNeed:
+        if self.fused:
+            return CacheNeed("state", state_shape=(K.delta_slot(*self.sizes, self.taps),), state_dtype=torch.float32)
+        return super().cache_need()
 
     def tensor_specs(self) -> List[TensorSpec]:
         H, nh = self.hidden_size, self.num_heads
@@ -162,17 +177,36 @@ class GatedDeltaRule(_RecurrentMixer):
 
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         t = lambda n: tensors[self.name(n)]
-        # q | k | v | gate in one product; the write strengths' and decays' logits (floats) in another
-        self.w_in = torch.cat([t("q"), t("k"), t("v"), t("gate")], dim=0).contiguous()
-        self.w_gates = torch.cat([t("write"), t("decay")], dim=0).contiguous()
-        self.w_conv = torch.cat([t("q_conv"), t("k_conv"), t("v_conv")], dim=0).contiguous()
-        self.a_log, self.dt_bias, self.gain = t("a_log"), t("dt_bias"), t("norm")
+        filters = torch.cat([t("q_conv"), t("k_conv"), t("v_conv")], dim=0)
+        if self.fused:
+            # everything in one product, filled up with zero rows to a whole number of the product kernels' tiles
+            rows = [t(n) for n in ("q", "k", "v", "gate", "write", "decay")]
+            n = sum(r.shape[0] for r in rows)
+            rows.append(torch.zeros((-n % 16, self.hidden_size), dtype=rows[0].dtype, device=rows[0].device))
+            self.w_in = torch.cat(rows, dim=0).contiguous()
+            self.w_conv = filters.T.contiguous()                          # by tap
+        else:
+            # q | k | v | gate in one product; the write strengths' and decays' logits (floats) in another
+            self.w_in = torch.cat([t("q"), t("k"), t("v"), t("gate")], dim=0).contiguous()
+            self.w_gates = torch.cat([t("write"), t("decay")], dim=0).contiguous()
+            self.w_conv = filters.contiguous()
+        self.a_log, self.dt_bias, self.gain = t("a_log").contiguous(), t("dt_bias").contiguous(), t("norm").contiguous()
         self.w_out = t("out")
         if self.out_scale:
             self.w_out, _ = fold_output_scale(self.w_out, None, t("out_scale"))
 
-    def forward(self, x_t: torch.Tensor, residual32: torch.Tensor, ctx, cache, write: bool = True) -> torch.Tensor:
+    def forward(self, x_t: torch.Tensor, residual32: Optional[torch.Tensor], ctx, cache, write: bool = True) -> torch.Tensor:
+        """residual32 + mix(x_t) (``residual32`` None: the second alone)."""
         self._check(write)
+        y = self._fused(x_t, ctx, cache) if self.fused else self._by_scan(x_t, ctx, cache)
+        return K.gemm(y, self.w_out, residual=residual32, out_f32=True)
+
+    def _fused(self, x_t, ctx, cache):
+        return K.delta_rule(K.gemm(x_t, self.w_in, out_f32=True), self.w_conv, self.a_log, self.dt_bias, self.gain, cache.state,
+                            (ctx.token_item, ctx.positions, ctx.item_len, ctx.item_tok_off, ctx.item_slot), *self.sizes,
+                            self.eps, self.unit_eps, self.dtype, all_single=bool(ctx.all_single))
+
+    def _by_scan(self, x_t, ctx, cache):
         qk, c = self.qk_size, self.conv_channels
         items = (ctx.token_item, ctx.item_len, ctx.item_tok_off, ctx.item_slot)
         conv_state, state = self._states(cache)
@@ -185,5 +219,4 @@ class GatedDeltaRule(_RecurrentMixer):
         K.unit_norm(qkv[:, qk:2 * qk], self.num_qk_heads, self.unit_eps)
         o = K.state_scan(qkv[:, :qk], qkv[:, qk:2 * qk], qkv[:, 2 * qk:], strength, decay, state, items,
                          self.num_heads, "delta", max_item_rows=1 if ctx.all_single else 0)
-        y = K.gated_group_norm(o, proj[:, c:], self.gain, self.num_heads, self.eps, self.dtype)
-        return K.gemm(y, self.w_out, residual=residual32, out_f32=True)
+        return K.gated_group_norm(o, proj[:, c:], self.gain, self.num_heads, self.eps, self.dtype)

@@ -211,7 +211,8 @@ def test_configuration_round_trip_spec_and_caches(name):
         if L["type"] == "delta":
             G, H = m["kv_heads"], m["heads"]
             assert needs[i].kind == "state"
-            assert needs[i].state_shape[0] >= m["conv"] * (2 * G * m["dim"] + H * m["vdim"]) + H * m["dim"] * m["vdim"]
+            inputs = m["conv"] if m["vdim"] <= 256 else m["conv"] - 1       # (a ring, or the last ones, of the filter)
+            assert needs[i].state_shape[0] >= inputs * (2 * G * m["dim"] + H * m["vdim"]) + H * m["dim"] * m["vdim"]
         elif m.get("kv_from") is None:
             assert e.write and needs[i].kind == "paged_kv" and needs[i].num_kv_heads == 1 and not needs[i].values
             assert needs[i].head_dim % 16 == 0 and needs[i].head_dim >= m["kv_rank"] + m["rot_dim"] and not needs[i].window
@@ -245,7 +246,8 @@ def test_configuration_errors_name_the_key():
         return str(e.value)
     assert "layers[0].mixer.heads" in broken(lambda c: c["layers"][0]["mixer"].update(heads=3))
     assert "conv" in broken(lambda c: c["layers"][0]["mixer"].update(conv=9))
-    assert "vdim" in broken(lambda c: c["layers"][0]["mixer"].update(vdim=300))
+    assert "dim" in broken(lambda c: c["layers"][0]["mixer"].update(dim=300))
+    assert "vdim" in broken(lambda c: c["layers"][0]["mixer"].pop("vdim"))
     assert "q_rank" in broken(lambda c: c["layers"][1]["mixer"].pop("q_rank"))
     assert "scale" in broken(lambda c: c["layers"][1]["mixer"].pop("scale"))
     assert "rot_dim" in broken(lambda c: c["layers"][1]["mixer"].update(kv_rank=600))

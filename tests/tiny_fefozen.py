@@ -10,7 +10,8 @@ C: one query/key head for 3 heads, keys wider than values (72 x 40), one tap; 20
    turned part of 64 of which 24 turn; one expert a token, no identity experts.
 D: one head everywhere, nothing turned, a latent of 16; a borrowing layer beside its lender; three of five choices, three of
    them identity experts.
-E: 40 heads (more than 32) on a latent of 270 (entries past 256), two taps, values of 130 channels; no experts.
+E: 40 heads (more than 32) on a latent of 270 (entries past 256), two taps, values of 130 channels, and of 264, which the delta
+   rule's scan takes; no experts.
 """
 from __future__ import annotations
 
@@ -66,7 +67,8 @@ CONFIGS = {
               [_moe(_latent(2, 1, 16, 16, 16, 16, 0.5), 2, 3, 3, 16, 1.2), _dense(_latent(2, 1, 20, 8, 24, 16, 0.6, None, kv_from=0), 32),
                _moe(_delta(1, 1, 32, 32, 2), 2, 3, 3, 16, 0.9)]),
     "E": _cfg(59, 96, 1e-5,
-              [_dense(_latent(1, 40, 4, 4, 80, 270, 0.5, (16, 16, 200.0)), 64), _dense(_delta(2, 1, 8, 130, 2), 40)]),
+              [_dense(_latent(1, 40, 4, 4, 80, 270, 0.5, (16, 16, 200.0)), 64), _dense(_delta(2, 1, 8, 130, 2), 40),
+               _delta(2, 2, 12, 264, 3)]),
 }
 PAGE_SIZE = {"A": 4, "B": 2, "C": 16, "D": 8, "E": 12}
 
